@@ -945,9 +945,9 @@ int semipd_sigmoid_gate(void* x, int64_t x_ld, const void* gate, int64_t gate_ld
 /* x [rows, heads * head_width] <- x * sigmoid(gate[row, head]), fp32 arithmetic.  No reference counterpart. */
 int semipd_sigmoid_gate_heads(void* x, int64_t x_ld, const void* gate, int64_t gate_ld, int64_t rows, int64_t heads,
                               int64_t head_width, int dtype, void* stream);
-/* out (fp32 [num_tokens, width]) = embed[ids[t]] * scale. */
-int semipd_embed_stream(const int64_t* ids, const void* embed, float scale, int64_t num_tokens, float* out, int64_t width,
-                        int dtype, void* stream);
+/* out (fp32 [num_tokens, width]) = embed[ids[t]] * scale; copy (may be NULL): the same rows in `dtype`. */
+int semipd_embed_stream(const int64_t* ids, const void* embed, float scale, int64_t num_tokens, float* out, void* copy,
+                        int64_t width, int dtype, void* stream);
 /* stream (fp32 rows, in place) <- rms_norm(alpha * stream + layer_scale * y) * weight (y, layer_scale may be NULL); when out
  * is given it receives the new stream in `dtype`, or with shift_mu (batches of ONE row per request only) the token-shifted
  * stream s + (prev - s) * shift_mu, prev the request's row of `prev` (zeros when seq_lens[row] <= 1), which is then
@@ -992,6 +992,62 @@ int semipd_state_space(const void* proj, int64_t ld, int64_t z_off, int64_t x_of
                        int64_t conv_ld, const int64_t* state_indices, const int64_t* seq_lens, const int32_t* q_start,
                        const int32_t* q_len, int64_t batch, int64_t num_tokens, int num_heads, int groups, int state_size, int v_dim,
                        int taps, void* out, int64_t out_ld, int fused_decode, int dtype, void* stream);
+
+/* ------------------------------------------------------------------ */
+/* Norm of a sublayer's output in front of the sum, a window with      */
+/* pooled blocks behind it, turned values, matrix memory               */
+/* ------------------------------------------------------------------ */
+/* stream (fp32 rows, in place) += rms_norm(y) * (weight + weight_shift); out (may be NULL) receives the new stream in `dtype`,
+ * or with next_weight rms_norm(stream) * (next_weight + next_shift).  fp32 arithmetic.  No reference counterpart. */
+int semipd_outnorm_stream(const void* y, int64_t y_ld, float* stream, int64_t stream_ld, const void* weight, float weight_shift,
+                          float eps, const void* next_weight, float next_shift, float next_eps, void* out, int64_t out_ld,
+                          int64_t rows, int64_t width, int dtype, void* stream_handle);
+/* out (fp32 [rows, half, 2]) = (cos, sin) of positions[t] * freq[i] (fp32 product). */
+int semipd_angle_table(const int64_t* positions, const float* freq, int half, int64_t rows, float* out, void* stream);
+/* Rows of qkv hold q | k | v at columns 0, k_off, v_off (num_kv_heads 0: queries only).  Every head of q and k: RMS norm times
+ * q_weight / k_weight [qk_dim], the first rot_dims elements turned in pairs (i, i + rot_dims / 2) by qk_angles (rows of
+ * semipd_angle_table); every head of v turned over all v_dim elements in pairs (m, m + v_dim / 2) by v_angles (NULL: v passes).
+ * q in place, k and v into the pools at loc.  pool > 0: also the mean key and value of every block of `pool` tokens
+ * (counted from the start of a sequence) that the batch completes, as semipd_block_means. */
+int semipd_head_norm_rope_kv_store(void* qkv, int64_t ld, int64_t num_tokens, int num_q_heads, int num_kv_heads, int qk_dim,
+                                   int v_dim, int64_t k_off, int64_t v_off, const void* q_weight, const void* k_weight, float eps,
+                                   const float* qk_angles, int rot_dims, const float* v_angles, void* k_pool, void* v_pool,
+                                   const int64_t* loc, const int64_t* positions, int pool, void* k_means, void* v_means, int k_piece,
+                                   int v_piece, const int32_t* req_to_token, int64_t req_to_token_stride,
+                                   const int64_t* req_pool_indices, const int64_t* seq_lens, const int32_t* q_start,
+                                   const int32_t* q_len, int64_t batch, int dtype, void* stream);
+/* The means of the blocks of `pool` tokens that the batch's rows complete, over the rows the pools hold, fp32 sums in token
+ * order, one rounding.  A mean is cut into pieces of k_piece / v_piece elements (powers of two, >= 8, piece * pool >= the head
+ * size); piece i of block b lies at the slot of token b * pool + i: k_means [slots, num_kv_heads, k_piece], v_means likewise. */
+int semipd_block_means(const void* k_pool, const void* v_pool, int num_kv_heads, int qk_dim, int v_dim, int pool, void* k_means,
+                       void* v_means, int k_piece, int v_piece, const int32_t* req_to_token, int64_t req_to_token_stride,
+                       const int64_t* req_pool_indices, const int64_t* seq_lens, const int32_t* q_start, const int32_t* q_len,
+                       int64_t batch, int64_t num_tokens, int dtype, void* stream);
+/* Sliding-window softmax attention (last `window` positions, 0: all) that sees, in the same softmax, the means of the blocks of
+ * `pool` tokens whose last token is at least `window` back (pool 0: none); sink as in semipd_local_attention.  The result of a
+ * head is turned back by `turn` ([rows, v_dim / 2, 2], pairs (m, m + v_dim / 2); NULL: not) and multiplied by
+ * sigmoid(gate[row, head]) (NULL: not).  n_splits / partial as in semipd_latent_attention (partial fp32
+ * [rows, heads, n_splits, v_dim + 2]). */
+int semipd_pooled_window_attention(const void* q, int64_t q_ld, const void* gate, int64_t gate_ld, void* out, int64_t out_ld,
+                                   const void* k_pool, const void* v_pool, const void* k_means, const void* v_means, int k_piece,
+                                   int v_piece, const int32_t* req_to_token, int64_t req_to_token_stride,
+                                   const int64_t* req_pool_indices, const int64_t* seq_lens, const int32_t* q_start,
+                                   const int32_t* q_len, int64_t batch, int64_t num_tokens, int64_t max_q_len, int num_q_heads,
+                                   int num_kv_heads, int qk_dim, int v_dim, float scale, int window, int pool, const float* sink,
+                                   const float* turn, int n_splits, float* partial, int form, int dtype, void* stream);
+/* fp32 elements of a work row and of a request's state of semipd_matrix_memory. */
+int64_t semipd_matrix_memory_work_width(int num_heads, int v_dim);
+int64_t semipd_matrix_memory_state_width(int num_heads, int qk_dim, int v_dim);
+/* Matrix memory with exponential gates behind its projection GEMM: rows [q | k | v | g | i | f] at the given columns, gate
+ * biases fp32 [H], norm_w [H * v_dim]; state fp32 [slots, state width] (S [H, qk_dim, v_dim] | n [H, qk_dim] | m [H]) is a column
+ * range of the requests' state rows; out [T, H * v_dim] = every head's read-out at unit RMS * norm_w * sigmoid(g).  Batch
+ * description as in semipd_local_attention.  form: 0 by shape and type, 1 token by token, 2 the matrix-core form. */
+int semipd_matrix_memory(const void* proj, int64_t ld, int64_t q_off, int64_t k_off, int64_t v_off, int64_t g_off, int64_t i_off,
+                         int64_t f_off, const float* i_bias, const float* f_bias, float gate_cap, const void* norm_w, float eps,
+                         float* work, int64_t work_ld, float* state, int64_t state_ld, const int64_t* state_indices,
+                         const int64_t* seq_lens, const int32_t* q_start, const int32_t* q_len, int64_t batch, int64_t num_tokens,
+                         int num_heads, int qk_dim, int v_dim, float q_scale, void* out, int64_t out_ld, int form, int dtype,
+                         void* stream);
 
 #ifdef __cplusplus
 }

@@ -417,13 +417,122 @@ __global__ void __launch_bounds__(256) sigmoid_gate_heads_kernel(T* __restrict__
   }
 }
 
-// ---- token embedding times a scale as the start of an fp32 stream
+// ---- token embedding times a scale as the start of an fp32 stream (`copy`: the same rows in the activation type, for a first
+// sublayer that reads the stream as it is)
 template <typename T>
 __global__ void __launch_bounds__(256) embed_stream_kernel(const int64_t* __restrict__ ids, const T* __restrict__ embed, float scale,
-                                                           float* __restrict__ out, int64_t width) {
+                                                           float* __restrict__ out, T* __restrict__ copy, int64_t width) {
   const int64_t t = blockIdx.x;
   const T* e = embed + ids[t] * width;
-  for (int64_t i = threadIdx.x; i < width; i += 256) out[t * width + i] = Elem<T>::to_f(e[i]) * scale;
+  for (int64_t i = threadIdx.x; i < width; i += 256) {
+    const float x = Elem<T>::to_f(e[i]) * scale;
+    out[t * width + i] = x;
+    if (copy) copy[t * width + i] = Elem<T>::from_f(x);
+  }
+}
+
+// ---- norm of a sublayer's OUTPUT in front of the sum on an fp32 stream:
+//     stream <- stream + y / sqrt(mean(y^2) + eps) * (weight + shift)                                  (fp32, in place)
+// and, when `out` is given, what comes next reads, in the activation type: the new stream itself, or -- with `w2` -- the new
+// stream / sqrt(mean(stream^2) + eps2) * (w2 + shift2), the norm in front of the vocabulary head.  A workgroup per row; VEC: the
+// row (at most 256 * 8 * NP elements) stays in registers, 16-byte accesses.
+template <typename T> __device__ __forceinline__ void load8f(const T* p, float (&f)[8]) {
+  if constexpr (sizeof(T) == 2) {
+    const Vec16<T> v = load16(p);
+#pragma unroll
+    for (int u = 0; u < 8; ++u) f[u] = Elem<T>::to_f(v.e[u]);
+  } else {
+    const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>((const float*)p + 4);
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+  }
+}
+template <typename T> __device__ __forceinline__ void store8f(T* p, const float (&f)[8]) {
+  if constexpr (sizeof(T) == 2) {
+    Vec16<T> v;
+#pragma unroll
+    for (int u = 0; u < 8; ++u) v.e[u] = Elem<T>::from_f(f[u]);
+    store16(p, v);
+  } else {
+    *reinterpret_cast<float4*>(p) = float4{f[0], f[1], f[2], f[3]};
+    *reinterpret_cast<float4*>((float*)p + 4) = float4{f[4], f[5], f[6], f[7]};
+  }
+}
+
+template <typename T, int NP>
+__global__ void __launch_bounds__(256) outnorm_stream_vec_kernel(const T* __restrict__ y, int64_t y_ld, float* __restrict__ stream,
+                                                                 int64_t s_ld, const T* __restrict__ w, float shift, float eps,
+                                                                 const T* __restrict__ w2, float shift2, float eps2,
+                                                                 T* __restrict__ out, int64_t out_ld, int64_t width) {
+  __shared__ float red[16];
+  const int64_t r = blockIdx.x;
+  float v[NP][8], x[NP][8], q = 0.f;
+#pragma unroll
+  for (int k = 0; k < NP; ++k) {
+    const int64_t i = ((int64_t)k * blockDim.x + threadIdx.x) * 8;
+#pragma unroll
+    for (int u = 0; u < 8; ++u) v[k][u] = 0.f;
+    if (i < width) {
+      load8f(y + r * y_ld + i, v[k]);
+      load8f(stream + r * s_ld + i, x[k]);
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u) q += v[k][u] * v[k][u];
+  }
+  const float rs = 1.0f / sqrtf(block_sum(q, red) / (float)width + eps);
+  float q2 = 0.f;
+#pragma unroll
+  for (int k = 0; k < NP; ++k) {
+    const int64_t i = ((int64_t)k * blockDim.x + threadIdx.x) * 8;
+    if (i >= width) continue;
+    float ww[8];
+    load8f(w + i, ww);
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      x[k][u] += v[k][u] * rs * (ww[u] + shift);
+      q2 += x[k][u] * x[k][u];
+    }
+    store8f(stream + r * s_ld + i, x[k]);
+    if (out && !w2) store8f(out + r * out_ld + i, x[k]);
+  }
+  if (!out || !w2) return;
+  const float rs2 = 1.0f / sqrtf(block_sum(q2, red) / (float)width + eps2);
+#pragma unroll
+  for (int k = 0; k < NP; ++k) {
+    const int64_t i = ((int64_t)k * blockDim.x + threadIdx.x) * 8;
+    if (i >= width) continue;
+    float ww[8];
+    load8f(w2 + i, ww);
+#pragma unroll
+    for (int u = 0; u < 8; ++u) x[k][u] *= rs2 * (ww[u] + shift2);
+    store8f(out + r * out_ld + i, x[k]);
+  }
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256) outnorm_stream_kernel(const T* __restrict__ y, int64_t y_ld, float* __restrict__ stream,
+                                                             int64_t s_ld, const T* __restrict__ w, float shift, float eps,
+                                                             const T* __restrict__ w2, float shift2, float eps2, T* __restrict__ out,
+                                                             int64_t out_ld, int64_t width) {
+  __shared__ float red[16];
+  const int64_t r = blockIdx.x;
+  float* x = stream + r * s_ld;
+  float q = 0.f;
+  for (int64_t i = threadIdx.x; i < width; i += 256) {
+    const float v = Elem<T>::to_f(y[r * y_ld + i]);
+    q += v * v;
+  }
+  const float rs = 1.0f / sqrtf(block_sum(q, red) / (float)width + eps);
+  float q2 = 0.f;
+  for (int64_t i = threadIdx.x; i < width; i += 256) {
+    const float v = x[i] + Elem<T>::to_f(y[r * y_ld + i]) * rs * (Elem<T>::to_f(w[i]) + shift);
+    x[i] = v;
+    q2 += v * v;
+    if (out && !w2) out[r * out_ld + i] = Elem<T>::from_f(v);
+  }
+  if (!out || !w2) return;
+  const float rs2 = 1.0f / sqrtf(block_sum(q2, red) / (float)width + eps2);
+  for (int64_t i = threadIdx.x; i < width; i += 256)           // (every thread re-reads the elements it wrote itself)
+    out[r * out_ld + i] = Elem<T>::from_f(x[i] * rs2 * (Elem<T>::to_f(w2[i]) + shift2));
 }
 
 // The request that owns row t of a batch, the row's index in the request's portion, the portion's length and the position
@@ -712,15 +821,40 @@ extern "C" int semipd_sigmoid_gate_heads(void* x, int64_t x_ld, const void* gate
   return launch_status("sigmoid_gate_heads");
 }
 
-extern "C" int semipd_embed_stream(const int64_t* ids, const void* embed, float scale, int64_t num_tokens, float* out, int64_t width,
-                                   int dtype, void* stream) {
+extern "C" int semipd_embed_stream(const int64_t* ids, const void* embed, float scale, int64_t num_tokens, float* out, void* copy,
+                                   int64_t width, int dtype, void* stream) {
   SEMIPD_CHECK_ARG(num_tokens >= 0 && width > 0, SEMIPD_EINVAL, "embed_stream: bad sizes");
   if (num_tokens == 0) return 0;
   SEMIPD_CHECK_ARG(ids && embed && out, SEMIPD_EINVAL, "embed_stream: null pointer");
   SEMIPD_DISPATCH_DTYPE(dtype, T,
                         hipLaunchKernelGGL((embed_stream_kernel<T>), dim3((unsigned)num_tokens), dim3(256), 0, as_stream(stream), ids,
-                                           (const T*)embed, scale, out, width));
+                                           (const T*)embed, scale, out, (T*)copy, width));
   return launch_status("embed_stream");
+}
+
+extern "C" int semipd_outnorm_stream(const void* y, int64_t y_ld, float* stream, int64_t stream_ld, const void* weight,
+                                     float weight_shift, float eps, const void* next_weight, float next_shift, float next_eps,
+                                     void* out, int64_t out_ld, int64_t rows, int64_t width, int dtype, void* stream_handle) {
+  SEMIPD_CHECK_ARG(rows >= 0 && width > 0, SEMIPD_EINVAL, "outnorm_stream: bad sizes");
+  if (rows == 0) return 0;
+  SEMIPD_CHECK_ARG(y && stream && weight && (!next_weight || out), SEMIPD_EINVAL,
+                   "outnorm_stream: null pointer, or a second norm without an output");
+  const int64_t esz = dtype == SEMIPD_F32 ? 4 : 2;
+  const bool vec = width % 8 == 0 && width <= 256 * 8 * 4 && aligned16(y) && (y_ld * esz) % 16 == 0 && aligned16(stream) &&
+                   stream_ld % 4 == 0 && aligned16(weight) && (!next_weight || aligned16(next_weight)) &&
+                   (!out || (aligned16(out) && (out_ld * esz) % 16 == 0));
+#define SEMIPD_OUTNORM(K)                                                                                                     \
+  hipLaunchKernelGGL((K), dim3((unsigned)rows), dim3(threads), 0, as_stream(stream_handle), (const T*)y, y_ld, stream, stream_ld,  \
+                     (const T*)weight, weight_shift, eps, (const T*)next_weight, next_shift, next_eps, (T*)out, out_ld, width)
+  SEMIPD_DISPATCH_DTYPE(dtype, T, {
+    const unsigned threads = !vec || width >= 2048 ? 256u : (unsigned)((width / 8 + 63) / 64 * 64);
+    if (!vec) SEMIPD_OUTNORM(outnorm_stream_kernel<T>);
+    else if (width <= 256 * 8) SEMIPD_OUTNORM((outnorm_stream_vec_kernel<T, 1>));
+    else if (width <= 256 * 8 * 2) SEMIPD_OUTNORM((outnorm_stream_vec_kernel<T, 2>));
+    else SEMIPD_OUTNORM((outnorm_stream_vec_kernel<T, 4>));
+  });
+#undef SEMIPD_OUTNORM
+  return launch_status("outnorm_stream");
 }
 
 extern "C" int semipd_postnorm_stream(const void* y, int64_t y_ld, const void* layer_scale, float* stream, int64_t stream_ld,

@@ -482,7 +482,21 @@ struct LocalAttnArgs {
   int n_splits;                    // decode form: workgroups that share the keys of one (request, kv head, 16 q heads) (0 / 1: one)
   float* partial;                  // [rows, H, n_splits, E + 2] fp32: unnormalised sums, running maximum, denominator
   int v_shared;                    // 1: the value row of a slot is ONE head of E elements that every key/value head's queries read
+  // block means (POOL kernels): blocks of `pool` tokens that lie wholly in front of the window are seen through one key and
+  // one value each.  The mean of block b is cut into pieces of 2^k_sh (2^v_sh) elements; piece i lies in the mean pools at the
+  // slot of token b * pool + i (rows of kb_ld / vb_ld elements, kv head g's piece at g << k_sh)
+  int pool;                        // 0: no blocks
+  const void* kb_pool; const void* vb_pool;
+  int64_t kb_ld, vb_ld;
+  int k_sh, v_sh;
+  const float* turn;               // POOL kernels: [rows, E / 2] (cos, sin): the result is turned BACK by these angles, pairs (m, m + E / 2)
 };
+
+// how many blocks a query at pos sees: those whose last token is at least `window` back
+__device__ __forceinline__ int64_t blocks_seen(const LocalAttnArgs& a, int64_t pos) {
+  const int64_t out = pos - a.window + 1;          // tokens in front of the window
+  return (a.pool > 0 && a.window > 0 && out > 0) ? out / a.pool : 0;
+}
 
 // first visible position of the contiguous range that ends at the query (the kept first positions come on top)
 __device__ __forceinline__ int64_t range_lo(const LocalAttnArgs& a, int64_t pos) {
@@ -519,7 +533,7 @@ __device__ __forceinline__ bool locate_row(const LocalAttnArgs& a, int64_t t, in
 }
 
 // ------------------------------------------------------------------------------------------------ one wave per row
-template <typename T, int NA>      // head sizes up to 64 * NA
+template <typename T, int NA, bool POOL>      // head sizes up to 64 * NA
 __global__ void __launch_bounds__(256) local_attention_rows_kernel(LocalAttnArgs a) {
   __shared__ float q_lds[4][64 * NA];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -544,15 +558,36 @@ __global__ void __launch_bounds__(256) local_attention_rows_kernel(LocalAttnArgs
 #pragma unroll
   for (int u = 0; u < NA; ++u) acc[u] = 0.f;
   constexpr int V = Elem<T>::kVec;
-  // the kept first positions (none without a window), then the range that ends at the query
-  for (int seg = n_first > 0 ? 0 : 1; seg < 2; ++seg) {
-    const int64_t j_begin = seg == 0 ? 0 : lo, j_last = seg == 0 ? n_first - 1 : pos;
+  // the kept first positions (none without a window) or the block means, then the range that ends at the query
+  const int64_t n_blocks = POOL ? blocks_seen(a, pos) : 0;
+  const T* kb = POOL ? (const T*)a.kb_pool + ((int64_t)g << a.k_sh) : nullptr;
+  const T* vb = POOL ? (const T*)a.vb_pool + ((int64_t)g << a.v_sh) : nullptr;
+  for (int seg = (n_first > 0 || n_blocks > 0) ? 0 : 1; seg < 2; ++seg) {
+    const bool blk = POOL && seg == 0;
+    const int64_t j_begin = seg == 0 ? 0 : lo, j_last = seg == 0 ? (POOL ? n_blocks : n_first) - 1 : pos;
     for (int64_t j0 = j_begin; j0 <= j_last; j0 += 64) {
       const int64_t j = j0 + lane;
       const bool valid = j <= j_last;
-      const int slot = valid ? row[j] : 0;
+      const int slot = valid && !blk ? row[j] : 0;
       float s = -INFINITY;
-      if (valid) {
+      if (POOL && blk) {
+        if (valid) {
+          const int32_t* brow = row + j * a.pool;
+          const int kmask = (1 << a.k_sh) - 1;
+          float dot = 0.f;
+          if ((D % V) == 0) {
+            for (int d = 0; d < D; d += V) {
+              const Vec16<T> kv = load16(kb + (int64_t)brow[d >> a.k_sh] * a.kb_ld + (d & kmask));
+#pragma unroll
+              for (int u = 0; u < V; ++u) dot += q_lds[wave][d + u] * Elem<T>::to_f(kv.e[u]);
+            }
+          } else {
+            for (int d = 0; d < D; ++d)
+              dot += q_lds[wave][d] * Elem<T>::to_f(kb[(int64_t)brow[d >> a.k_sh] * a.kb_ld + (d & kmask)]);
+          }
+          s = capped(dot, a.scale, a.cap);
+        }
+      } else if (valid) {
         const T* k = kp + (int64_t)slot * a.k_ld + (int64_t)g * D;
         float dot = 0.f;
         if ((D % V) == 0) {
@@ -582,6 +617,16 @@ __global__ void __launch_bounds__(256) local_attention_rows_kernel(LocalAttnArgs
       for (int jj = 0; jj < n; ++jj) {
         const float pj = __shfl(p, jj, 64);
         const int sj = __shfl(slot, jj, 64);
+        if (POOL && blk) {
+          const int32_t* brow = row + (j0 + jj) * a.pool;
+          const int vmask = (1 << a.v_sh) - 1;
+#pragma unroll
+          for (int u = 0; u < NA; ++u) {
+            const int e = lane + 64 * u;
+            if (e < E) acc[u] += pj * Elem<T>::to_f(vb[(int64_t)brow[e >> a.v_sh] * a.vb_ld + (e & vmask)]);
+          }
+          continue;
+        }
         const T* v = vp + (int64_t)sj * a.v_ld + (a.v_shared ? 0 : (int64_t)g * E);
 #pragma unroll
         for (int u = 0; u < NA; ++u) {
@@ -594,6 +639,30 @@ __global__ void __launch_bounds__(256) local_attention_rows_kernel(LocalAttnArgs
   if (!sig && a.sink != nullptr) l += expf(a.sink[h] - m);
   const float inv = sig ? a.out_scale : a.out_scale / l;
   T* o = (T*)a.out + t * a.out_ld + (int64_t)h * E;
+  if constexpr (POOL) {          // turned back, pairs (m, m + E / 2), and one gate per head
+    const float gv = a.gate ? 1.0f / (1.0f + expf(-Elem<T>::to_f(((const T*)a.gate)[t * a.gate_ld + h]))) : 1.0f;
+    const int half = E >> 1;
+    const float2* cs = reinterpret_cast<const float2*>(a.turn) + t * half;
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int u = 0; u < NA; ++u) {
+      const int e = lane + 64 * u;
+      if (e < E) q_lds[wave][e] = acc[u] * inv;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    for (int e = lane; e < E; e += 64) {
+      float y = q_lds[wave][e];
+      if (a.turn) {
+        const float2 c = cs[e < half ? e : e - half];
+        y = e < half ? y * c.x + q_lds[wave][e + half] * c.y : y * c.x - q_lds[wave][e - half] * c.y;
+      }
+      o[e] = Elem<T>::from_f(y * gv);
+    }
+    return;
+  }
   const T* gt = a.gate ? (const T*)a.gate + t * a.gate_ld + (int64_t)h * E : nullptr;
 #pragma unroll
   for (int u = 0; u < NA; ++u) {
@@ -613,16 +682,6 @@ __global__ void __launch_bounds__(256) local_attention_rows_kernel(LocalAttnArgs
 // O^T += V^T P^T once the a operand numbers its k slots the same way: V^T comes out of a row-major LDS tile [32][E] through
 // the transposing read ds_read_b64_tr_b16, four keys x 16 value elements per 16-lane group.
 // The loads of step i + 1 (K fragments, V rows) are in flight in registers while step i is multiplied.
-typedef float f32x4 __attribute__((ext_vector_type(4)));
-
-template <typename T> __device__ __forceinline__ f32x4 mma16(const Frag16& a, const Frag16& b, f32x4 c);
-template <> __device__ __forceinline__ f32x4 mma16<bf16_t>(const Frag16& a, const Frag16& b, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, b.b, c, 0, 0, 0);
-}
-template <> __device__ __forceinline__ f32x4 mma16<f16_t>(const Frag16& a, const Frag16& b, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x32_f16(a.f, b.f, c, 0, 0, 0);
-}
-
 // Scores live in the base-2 domain (multiplied by log2 e) so that every exponential is one v_exp_f32, and the cap is
 //   cap * tanh(x / cap) * log2e = A - 2 A / (exp2(c raw) + 1),  A = cap log2e,  c = 2 scale log2e / cap
 // (one exp, one reciprocal: exp2 overflow gives A, underflow -A).  Without a cap: raw * scale * log2e.
@@ -652,6 +711,51 @@ template <int ND> struct KFrags {
   Frag16 a[ND], b[ND];
 };
 
+// Where the rows of key j lie.  TokenRows: key j is position j of the sequence, its slot from the copy of this part of the
+// request's row in LDS when the caller made one (the load of a row of the pool then waits for nothing but itself), else from
+// the table.
+template <typename T> struct TokenRows {
+  const T* kp; int64_t kstride;
+  const T* vp; int64_t vstride;
+  const int32_t* row; const int32_t* idx_lds; int64_t idx_base;
+  __device__ __forceinline__ int64_t slot(int64_t j) const { return idx_lds ? idx_lds[j - idx_base] : row[j]; }
+  __device__ __forceinline__ bool have(int64_t j, int64_t j_end) const { return j <= j_end; }
+  __device__ __forceinline__ const T* k(int64_t j, int e) const { return kp + slot(j) * kstride + e; }
+  __device__ __forceinline__ const T* v(int64_t j, int e) const { return vp + slot(j) * vstride + e; }
+  // a lane's K row: looked up once for all of its pieces (keys that are not there: the dummy slot)
+  struct KRow {
+    const T* p;
+    __device__ __forceinline__ const T* at(int e) const { return p + e; }
+  };
+  __device__ __forceinline__ KRow krow(int64_t j, int64_t j_end) const { return KRow{kp + (j <= j_end ? slot(j) : 0) * kstride}; }
+};
+// PooledRows: keys 0 .. nb - 1 are the block means (nb_pad: nb up to whole steps of 32 keys, so that a step is all blocks or
+// all tokens), key nb_pad + i is position tok0 + i.
+template <typename T> struct PooledRows {
+  TokenRows<T> tok;
+  const T* kb; int64_t kb_ld;
+  const T* vb; int64_t vb_ld;
+  int k_sh, v_sh, pool;
+  int64_t nb, nb_pad, tok0;
+  __device__ __forceinline__ bool have(int64_t j, int64_t j_end) const { return j < nb_pad ? j < nb : j <= j_end; }
+  __device__ __forceinline__ const T* k(int64_t j, int e) const {
+    if (j < nb_pad) return kb + tok.slot(j * pool + (e >> k_sh)) * kb_ld + (e & ((1 << k_sh) - 1));
+    return tok.k(tok0 + j - nb_pad, e);
+  }
+  __device__ __forceinline__ const T* v(int64_t j, int e) const {
+    if (j < nb_pad) return vb + tok.slot(j * pool + (e >> v_sh)) * vb_ld + (e & ((1 << v_sh) - 1));
+    return tok.v(tok0 + j - nb_pad, e);
+  }
+  struct KRow {
+    const PooledRows* r; int64_t j; const T* p;      // p: the row of a token, null for a block
+    __device__ __forceinline__ const T* at(int e) const { return p ? p + e : r->k(j, e); }
+  };
+  __device__ __forceinline__ KRow krow(int64_t j, int64_t j_end) const {
+    if (!have(j, j_end)) return KRow{this, j, tok.kp};                      // the dummy slot
+    return j < nb_pad ? KRow{this, j, nullptr} : KRow{this, j, tok.k(tok0 + j - nb_pad, 0)};
+  }
+};
+
 // The walk over keys j_begin, j_begin + j_step, ... (steps of 32 keys, keys past j_end masked) for the 16 columns of this wave.
 //   NT threads (a workgroup with BLOCK_SYNC, else one wave) stage the V tile of every step; `tid` is the thread's index among
 //   them.  relevant(j0): whether this wave has anything to multiply in the step at j0 (it stages and syncs anyway).
@@ -660,12 +764,10 @@ template <int ND> struct KFrags {
 //   in whole rows; a wave on its own takes its K fragments straight from the pool into operand layout.
 //   32 keys per step (64 between one pair of barriers measured slower: the staging registers of 64 rows push the 128 / 128
 //   kernel into scratch).
-template <typename T, int ND, int NE, int NT, bool BLOCK_SYNC, bool SIG, typename Ok, typename Relevant>
-__device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[ND], int nd, int ne, int E, const T* kp,
-                                         int64_t kstride, const T* vp, int64_t vstride, const int32_t* row, int64_t j_begin,
-                                         int64_t j_end, int64_t j_step, uint8_t* v_lds, int tid, float scale, float cap, Ok ok,
-                                         Relevant relevant, int r, int g, const int32_t* idx_lds, int64_t idx_base,
-                                         float hb = 0.f) {
+template <typename T, int ND, int NE, int NT, bool BLOCK_SYNC, bool SIG, typename Rows, typename Ok, typename Relevant>
+__device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[ND], int nd, int ne, int E, const Rows& rows,
+                                         int64_t j_begin, int64_t j_end, int64_t j_step, uint8_t* v_lds, int tid, float scale,
+                                         float cap, Ok ok, Relevant relevant, int r, int g, float hb = 0.f) {
   constexpr int KS = 32;                          // keys per step
   constexpr int NV = (NE * 2 * KS) / NT;          // 16-byte pieces of V per thread and step, at most
   constexpr int NK = BLOCK_SYNC ? (ND * 4 * KS) / NT : 1;   // the same for K rows that go through LDS
@@ -692,9 +794,6 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
     k_key[i] = (BLOCK_SYNC && c < pieces_k) ? c / per_key_k : -1;
     k_ec[i] = (BLOCK_SYNC && c < pieces_k) ? c - k_key[i] * per_key_k : 0;
   }
-  // pool slot of key j: from the copy of this part of the request's row in LDS when the caller made one (the load of a row
-  // of the pool then waits for nothing but itself), else from the table
-  auto slot_of = [&](int64_t j) -> int64_t { return idx_lds ? idx_lds[j - idx_base] : row[j]; };
   auto sync = [&]() {
     if constexpr (BLOCK_SYNC) {
       __syncthreads();
@@ -709,7 +808,7 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
     for (int i = 0; i < NV; ++i)
       if (v_key[i] >= 0) {
         const int64_t j = j0 + v_key[i];
-        vr[i] = j <= j_end ? *reinterpret_cast<const uint4*>(vp + slot_of(j) * vstride + v_ec[i] * 8) : uint4{0u, 0u, 0u, 0u};
+        vr[i] = rows.have(j, j_end) ? *reinterpret_cast<const uint4*>(rows.v(j, v_ec[i] * 8)) : uint4{0u, 0u, 0u, 0u};
       }
   };
   auto store_v = [&](int buf) {        // buf: which pair of tiles (a lone wave has one)
@@ -727,18 +826,17 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
     for (int i = 0; i < NK; ++i)
       if (k_key[i] >= 0) {
         const int64_t j = j0 + k_key[i];
-        kr[i] = j <= j_end ? *reinterpret_cast<const uint4*>(kp + slot_of(j) * kstride + k_ec[i] * 8) : uint4{0u, 0u, 0u, 0u};
+        kr[i] = rows.have(j, j_end) ? *reinterpret_cast<const uint4*>(rows.k(j, k_ec[i] * 8)) : uint4{0u, 0u, 0u, 0u};
       }
   };
   auto load_k = [&](int64_t j0, auto& k) {
     const int64_t ja = j0 + r, jb = ja + 16;
-    const T* pa = kp + (ja <= j_end ? slot_of(ja) : 0) * kstride + 8 * g;
-    const T* pb = kp + (jb <= j_end ? slot_of(jb) : 0) * kstride + 8 * g;
+    const auto pa = rows.krow(ja, j_end), pb = rows.krow(jb, j_end);
 #pragma unroll
     for (int kk = 0; kk < ND; ++kk)
       if (kk < nd) {
-        k.a[kk].u = *reinterpret_cast<const uint4*>(pa + 32 * kk);
-        k.b[kk].u = *reinterpret_cast<const uint4*>(pb + 32 * kk);
+        k.a[kk].u = *reinterpret_cast<const uint4*>(pa.at(8 * g + 32 * kk));
+        k.b[kk].u = *reinterpret_cast<const uint4*>(pb.at(8 * g + 32 * kk));
       }
   };
   auto compute = [&](int64_t j0, const auto& k, int half, auto after_scores) {   // keys j0 .. j0 + 31 out of tile pair `half`
@@ -852,8 +950,8 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
 }
 
 // Prompt portions: 64 query rows of one request and one head per workgroup, 16 per wave.
-template <typename T, int ND, int NE, bool SIG>
-__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 4 ? 4 : 1))) local_attention_mfma_kernel(LocalAttnArgs a) {
+template <typename T, int ND, int NE, bool SIG, bool POOL>
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 4 ? (POOL ? 3 : 4) : 1))) local_attention_mfma_kernel(LocalAttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) uint8_t v_lds[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
   // Workgroup -> (kv head, 64-row tile, q head of the group), the last fastest.  Consecutive workgroup ids go round the
@@ -919,18 +1017,35 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 
   for (int eb = 0; eb < NE; ++eb) st.acc[eb] = f32x4{0.f, 0.f, 0.f, 0.f};
   const int32_t* row = a.req_to_token + a.req_pool_indices[b] * a.r2t_stride;
   const float hb = (SIG && a.head_bias) ? a.head_bias[h] * kLog2e : 0.f;
-  // the kept first positions that lie in front of the tile's window range: visible to every row of the tile
-  const int64_t n_first = keep < blk_lo ? keep : blk_lo;
-  if (n_first > 0)
+  const TokenRows<T> rows{(const T*)a.k_pool + (int64_t)gk * D, a.k_ld, (const T*)a.v_pool + (a.v_shared ? 0 : (int64_t)gk * E),
+                          a.v_ld, row, nullptr, 0};
+  if constexpr (POOL) {
+    // one walk: the blocks that the tile's last row sees, then the positions of the tile's window range
+    const int64_t nb = blocks_seen(a, blk_hi), nb_pad = (nb + 31) / 32 * 32;
+    const int64_t my_nb = blocks_seen(a, my_pos), w_nb = blocks_seen(a, w_hi);
+    const PooledRows<T> prows{rows, (const T*)a.kb_pool + ((int64_t)gk << a.k_sh), a.kb_ld,
+                              (const T*)a.vb_pool + ((int64_t)gk << a.v_sh), a.vb_ld, a.k_sh, a.v_sh, a.pool, nb, nb_pad, blk_lo};
+    key_walk<T, ND, NE, 256, true, false>(
+        st, qf, nd, ne, E, prows, 0, nb_pad + blk_hi - blk_lo, 32, v_lds, tid, a.scale, a.cap,
+        [&](int64_t j) {
+          const int64_t p = blk_lo + j - nb_pad;
+          return q_ok && (j < nb_pad ? j < my_nb : (p <= my_pos && p >= my_lo));
+        },
+        [&](int64_t j0) {
+          const int64_t p = blk_lo + j0 - nb_pad;
+          return wave_on && (j0 < nb_pad ? j0 < w_nb : (p <= w_hi && p + 31 >= w_lo));
+        }, r, g);
+  } else {
+    // the kept first positions that lie in front of the tile's window range: visible to every row of the tile
+    const int64_t n_first = keep < blk_lo ? keep : blk_lo;
+    if (n_first > 0)
+      key_walk<T, ND, NE, 256, true, SIG>(st, qf, nd, ne, E, rows, 0, n_first - 1, 32, v_lds, tid, a.scale, a.cap,
+                                          [&](int64_t j) { return q_ok && j < n_first; }, [&](int64_t) { return wave_on; }, r, g, hb);
     key_walk<T, ND, NE, 256, true, SIG>(
-        st, qf, nd, ne, E, (const T*)a.k_pool + (int64_t)gk * D, a.k_ld, (const T*)a.v_pool + (a.v_shared ? 0 : (int64_t)gk * E),
-        a.v_ld, row, 0, n_first - 1, 32, v_lds, tid, a.scale, a.cap, [&](int64_t j) { return q_ok && j < n_first; },
-        [&](int64_t) { return wave_on; }, r, g, nullptr, 0, hb);
-  key_walk<T, ND, NE, 256, true, SIG>(
-      st, qf, nd, ne, E, (const T*)a.k_pool + (int64_t)gk * D, a.k_ld, (const T*)a.v_pool + (a.v_shared ? 0 : (int64_t)gk * E),
-      a.v_ld, row, blk_lo, blk_hi, 32, v_lds, tid, a.scale, a.cap,
-      [&](int64_t j) { return q_ok && j <= my_pos && (j >= my_lo || j < keep); },
-      [&](int64_t j0) { return wave_on && j0 <= w_hi && (j0 + 31 >= w_lo || j0 < keep); }, r, g, nullptr, blk_lo, hb);
+        st, qf, nd, ne, E, rows, blk_lo, blk_hi, 32, v_lds, tid, a.scale, a.cap,
+        [&](int64_t j) { return q_ok && j <= my_pos && (j >= my_lo || j < keep); },
+        [&](int64_t j0) { return wave_on && j0 <= w_hi && (j0 + 31 >= w_lo || j0 < keep); }, r, g, hb);
+  }
   float l = st.l;
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
@@ -941,6 +1056,47 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 
   // 16-element block -- written out like that, rows would go to memory in 8-byte pieces; the wave lays its 16 x E tile down in
   // LDS and takes it up again in whole 16-byte pieces of consecutive lanes, so the gate is read and the result written in
   // full rows.
+  if constexpr (POOL) {
+    // fp32 through LDS: an element is turned back together with its partner half a head away, then the head's gate
+    const int ofs = E + 4;
+    float* of = reinterpret_cast<float*>(v_lds) + wave * 16 * ofs;
+#pragma unroll
+    for (int eb = 0; eb < NE; ++eb)
+      if (eb < ne)
+        *reinterpret_cast<float4*>(of + r * ofs + eb * 16 + 4 * g) =
+            float4{st.acc[eb][0] * inv, st.acc[eb][1] * inv, st.acc[eb][2] * inv, st.acc[eb][3] * inv};
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    const int per_row = E >> 3, half = E >> 1;
+    for (int c = lane; c < 16 * per_row; c += 64) {
+      const int rr = c / per_row, e0 = (c - rr * per_row) * 8;
+      if (wq0 + rr >= qn) continue;
+      const int64_t t = t0 + wq0 + rr;
+      const float gv = a.gate ? __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(
+                                    -kLog2e * Elem<T>::to_f(((const T*)a.gate)[t * a.gate_ld + h])))
+                              : 1.0f;
+      const float* x = of + rr * ofs + e0;
+      Vec16<T> v;
+      if (a.turn) {
+        const bool first = e0 < half;
+        const float* y = first ? x + half : x - half;
+        const float4* cs = reinterpret_cast<const float4*>(a.turn + (t * half + (first ? e0 : e0 - half)) * 2);
+        const float sg = first ? 1.0f : -1.0f;
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const float4 w = cs[u];            // (cos, sin) of two pairs
+          v.e[2 * u] = Elem<T>::from_f((x[2 * u] * w.x + sg * y[2 * u] * w.y) * gv);
+          v.e[2 * u + 1] = Elem<T>::from_f((x[2 * u + 1] * w.z + sg * y[2 * u + 1] * w.w) * gv);
+        }
+      } else {
+#pragma unroll
+        for (int u = 0; u < 8; ++u) v.e[u] = Elem<T>::from_f(x[u] * gv);
+      }
+      store16((T*)a.out + t * a.out_ld + (int64_t)h * E + e0, v);
+    }
+    return;
+  }
   const int ors = E * 2 + 16;
   uint8_t* o_lds = v_lds + wave * 16 * ors;
 #pragma unroll
@@ -971,10 +1127,27 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 
   }
 }
 
+// POOL forms of one row per request: elements first, first + step, ... of the result of head h (sum_of(e)) turned back in
+// pairs (m, m + E / 2), times the head's gate
+template <typename T, typename Sum>
+__device__ __forceinline__ void turned_back_store(const LocalAttnArgs& a, int64_t t, int h, T* o, int first, int step, Sum sum_of) {
+  const int half = a.E >> 1;
+  const float gv = a.gate ? __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(
+                                -kLog2e * Elem<T>::to_f(((const T*)a.gate)[t * a.gate_ld + h])))
+                          : 1.0f;
+  const float2* cs = reinterpret_cast<const float2*>(a.turn) + t * half;
+  for (int m = first; m < half; m += step) {
+    const float u = sum_of(m), v = sum_of(m + half);
+    const float2 c = a.turn ? cs[m] : float2{1.0f, 0.0f};
+    o[m] = Elem<T>::from_f((u * c.x + v * c.y) * gv);
+    o[m + half] = Elem<T>::from_f((v * c.x - u * c.y) * gv);
+  }
+}
+
 // Decode steps: one workgroup per (request, kv head, group of 16 q heads); the q heads are the 16 columns, the waves
 // take the 32-key steps in turn, each with a V tile of its own, and meet in LDS.
 // (eight waves for head sizes up to 128, four above: the walk's registers at 256 / 256 do not fit eight waves per CU)
-template <typename T, int ND, int NE, int NW, bool SIG>
+template <typename T, int ND, int NE, int NW, bool SIG, bool POOL>
 __global__ void __launch_bounds__(64 * NW) local_attention_decode_kernel(LocalAttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) uint8_t v_lds[];
   __shared__ float part_ml[NW][2][16];
@@ -993,8 +1166,16 @@ __global__ void __launch_bounds__(64 * NW) local_attention_decode_kernel(LocalAt
   const int64_t lo_q = range_lo(a, pos_q), n_first = split == 0 ? kept_before(a, lo_q) : 0;
   // with several workgroups per (request, kv head, 16 q heads) this one walks a slice of the range (whole 32-key steps; it
   // may be empty) and leaves unnormalised sums for the merge kernel
-  int64_t lo = lo_q, pos = pos_q;
-  if (n_splits > 1) {
+  // (POOL: the range is that of PooledRows' keys -- the blocks seen, then the positions of the window)
+  const int64_t nb = POOL ? blocks_seen(a, pos_q) : 0, nb_pad = (nb + 31) / 32 * 32;
+  int64_t lo = POOL ? 0 : lo_q, pos = POOL ? nb_pad + pos_q - lo_q : pos_q;
+  if (POOL && n_splits > 1) {
+    const int64_t last = pos;
+    int64_t chunk = (last + n_splits) / n_splits;
+    chunk = (chunk + 31) / 32 * 32;
+    lo = split * chunk;
+    pos = lo + chunk - 1 < last ? lo + chunk - 1 : last;
+  } else if (n_splits > 1) {
     int64_t chunk = (pos_q - lo_q + n_splits) / n_splits;
     chunk = (chunk + 31) / 32 * 32;
     lo = lo_q + split * chunk;
@@ -1018,22 +1199,36 @@ __global__ void __launch_bounds__(64 * NW) local_attention_decode_kernel(LocalAt
   const int tile_bytes = 32 * v_tile_row_bytes(E) > E * 17 * 4 ? 32 * v_tile_row_bytes(E) : E * 17 * 4;
   uint8_t* mine_b = v_lds + wave * tile_bytes;
   __shared__ int32_t idx_lds[kIdxLds];
-  const bool idx_fits = pos - lo < kIdxLds;
+  // positions whose slots this slice looks up
+  int64_t p_lo = lo, p_hi = pos;
+  if (POOL) {
+    p_lo = lo < nb_pad ? lo * a.pool : lo_q + lo - nb_pad;
+    p_hi = pos < nb_pad ? (pos < nb ? pos + 1 : nb) * a.pool - 1 : lo_q + pos - nb_pad;
+  }
+  const bool idx_fits = p_hi - p_lo < kIdxLds;
   if (idx_fits) {
-    for (int64_t j = lo + tid; j <= pos; j += 64 * NW) idx_lds[j - lo] = row[j];
+    for (int64_t j = p_lo + tid; j <= p_hi; j += 64 * NW) idx_lds[j - p_lo] = row[j];
     __syncthreads();
   }
   // (pos < lo: an empty slice; the walk below does nothing and the partial sums are those of no keys)
-  // the kept first positions in front of the window (none without one), then the range that ends at the query
-  if (n_first > 0)
-    key_walk<T, ND, NE, 64, false, SIG>(
-        st, qf, nd, ne, E, (const T*)a.k_pool + (int64_t)gk * D, a.k_ld, (const T*)a.v_pool + (a.v_shared ? 0 : (int64_t)gk * E),
-        a.v_ld, row, (int64_t)32 * wave, n_first - 1, 32 * NW, mine_b, lane, a.scale, a.cap,
-        [&](int64_t j) { return j < n_first; }, [&](int64_t) { return true; }, r, g, nullptr, 0, hb);
-  key_walk<T, ND, NE, 64, false, SIG>(
-      st, qf, nd, ne, E, (const T*)a.k_pool + (int64_t)gk * D, a.k_ld, (const T*)a.v_pool + (a.v_shared ? 0 : (int64_t)gk * E),
-      a.v_ld, row, lo + 32 * wave, pos, 32 * NW, mine_b, lane, a.scale, a.cap, [&](int64_t j) { return j <= pos; },
-      [&](int64_t) { return true; }, r, g, idx_fits ? idx_lds : nullptr, lo, hb);
+  const TokenRows<T> rows{(const T*)a.k_pool + (int64_t)gk * D, a.k_ld, (const T*)a.v_pool + (a.v_shared ? 0 : (int64_t)gk * E),
+                          a.v_ld, row, idx_fits ? idx_lds : nullptr, p_lo};
+  if constexpr (POOL) {
+    const PooledRows<T> prows{rows, (const T*)a.kb_pool + ((int64_t)gk << a.k_sh), a.kb_ld,
+                              (const T*)a.vb_pool + ((int64_t)gk << a.v_sh), a.vb_ld, a.k_sh, a.v_sh, a.pool, nb, nb_pad, lo_q};
+    key_walk<T, ND, NE, 64, false, false>(st, qf, nd, ne, E, prows, lo + 32 * wave, pos, 32 * NW, mine_b, lane, a.scale, a.cap,
+                                          [&](int64_t j) { return j < nb_pad ? j < nb && j <= pos : j <= pos; },
+                                          [&](int64_t) { return true; }, r, g);
+  } else {
+    // the kept first positions in front of the window (none without one), then the range that ends at the query
+    if (n_first > 0) {
+      const TokenRows<T> first{rows.kp, rows.kstride, rows.vp, rows.vstride, row, nullptr, 0};
+      key_walk<T, ND, NE, 64, false, SIG>(st, qf, nd, ne, E, first, (int64_t)32 * wave, n_first - 1, 32 * NW, mine_b, lane, a.scale,
+                                          a.cap, [&](int64_t j) { return j < n_first; }, [&](int64_t) { return true; }, r, g, hb);
+    }
+    key_walk<T, ND, NE, 64, false, SIG>(st, qf, nd, ne, E, rows, lo + 32 * wave, pos, 32 * NW, mine_b, lane, a.scale, a.cap,
+                                        [&](int64_t j) { return j <= pos; }, [&](int64_t) { return true; }, r, g, hb);
+  }
   float l = st.l;
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
@@ -1082,6 +1277,16 @@ __global__ void __launch_bounds__(64 * NW) local_attention_decode_kernel(LocalAt
   if (!SIG && a.sink != nullptr) lt += __builtin_amdgcn_exp2f(a.sink[hh] * kLog2e - m);
   const float inv = SIG ? a.out_scale : a.out_scale / lt;
   T* o = (T*)a.out + t * a.out_ld + (int64_t)hh * E;
+  if constexpr (POOL) {
+    auto sum_of = [&](int e) {
+      float y = 0.f;
+#pragma unroll
+      for (int w = 0; w < NW; ++w) y += f[w] * reinterpret_cast<const float*>(v_lds + w * tile_bytes)[e * 17 + c];
+      return y * inv;
+    };
+    turned_back_store<T>(a, t, hh, o, slice, 4 * NW, sum_of);
+    return;
+  }
   const T* gt = a.gate ? (const T*)a.gate + t * a.gate_ld + (int64_t)hh * E : nullptr;
   for (int e = slice; e < E; e += 4 * NW) {
     float y = 0.f;
@@ -1095,7 +1300,7 @@ __global__ void __launch_bounds__(64 * NW) local_attention_decode_kernel(LocalAt
 
 // The slices of a decode row's keys, each with its own running maximum (base-2 domain), denominator and unnormalised sums:
 // out = sum_s 2^(m_s - m) y_s / (sum_s 2^(m_s - m) l_s + 2^(sink log2 e - m)), a workgroup per (row, head).
-template <typename T, bool SIG>
+template <typename T, bool SIG, bool POOL>
 __global__ void __launch_bounds__(64) local_attention_merge_kernel(LocalAttnArgs a) {
   const int64_t b = blockIdx.x;
   const int h = blockIdx.y, E = a.E, n = a.n_splits;
@@ -1112,6 +1317,18 @@ __global__ void __launch_bounds__(64) local_attention_merge_kernel(LocalAttnArgs
   if (!SIG && a.sink != nullptr) lt += __builtin_amdgcn_exp2f(a.sink[h] * kLog2e - m);
   const float inv = SIG ? a.out_scale : a.out_scale / lt;
   T* o = (T*)a.out + t * a.out_ld + (int64_t)h * E;
+  if constexpr (POOL) {
+    auto sum_of = [&](int e) {
+      float y = 0.f;
+      for (int s = 0; s < n; ++s) {
+        const float ms = part[s * (E + 2) + E];
+        y += (ms == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(ms - m)) * part[s * (E + 2) + e];
+      }
+      return y * inv;
+    };
+    turned_back_store<T>(a, t, h, o, (int)threadIdx.x, 64, sum_of);
+    return;
+  }
   const T* gt = a.gate ? (const T*)a.gate + t * a.gate_ld + (int64_t)h * E : nullptr;
   for (int e = threadIdx.x; e < E; e += 64) {
     float y = 0.f;
@@ -1179,6 +1396,7 @@ extern "C" int semipd_unit_norm_kv_store(void* qkv, int64_t ld, int64_t num_toke
 }
 
 static int launch_local_attention(LocalAttnArgs a, int64_t max_q_len, int form, int dtype, void* stream);
+constexpr size_t kMaxDynLds = 96 * 1024;      // what the matrix-core forms may ask for (the attribute is set once per kernel)
 
 extern "C" int semipd_local_attention(const void* q, int64_t q_ld, const void* gate, int64_t gate_ld, void* out, int64_t out_ld,
                                       const void* k_pool, const void* v_pool, const int32_t* req_to_token,
@@ -1210,7 +1428,8 @@ extern "C" int semipd_window_attention(const void* q, int64_t q_ld, void* out, i
   return launch_local_attention(a, max_q_len, form, dtype, stream);
 }
 
-static int launch_local_attention(LocalAttnArgs a, int64_t max_q_len, int form, int dtype, void* stream) {
+template <bool POOL>
+static int launch_attention(LocalAttnArgs a, int64_t max_q_len, int form, int dtype, void* stream) {
   const void* q = a.q; const void* gate = a.gate; void* out = a.out; const void* k_pool = a.k_pool; const void* v_pool = a.v_pool;
   const int64_t q_ld = a.q_ld, gate_ld = a.gate_ld, out_ld = a.out_ld, batch = a.batch, num_tokens = a.num_tokens;
   const int32_t* q_start = a.q_start; const int32_t* q_len = a.q_len;
@@ -1231,12 +1450,13 @@ static int launch_local_attention(LocalAttnArgs a, int64_t max_q_len, int form, 
   const bool half = dtype == SEMIPD_BF16 || dtype == SEMIPD_F16;
   const bool mfma_ok = half && local_mfma_shape_ok(qk_dim, v_dim) && aligned16(q) && q_ld % 8 == 0 && aligned16(k_pool) &&
                        aligned16(v_pool) && a.k_ld % 8 == 0 && a.v_ld % 8 == 0 && aligned16(out) && out_ld % 8 == 0 &&
-                       (gate == nullptr || (aligned16(gate) && gate_ld % 8 == 0));
+                       (POOL || gate == nullptr || (aligned16(gate) && gate_ld % 8 == 0)) &&
+                       (!POOL || a.pool == 0 || (aligned16(a.kb_pool) && aligned16(a.vb_pool) && a.k_sh >= 3 && a.v_sh >= 3));
   SEMIPD_CHECK_ARG(form != 2 || mfma_ok, SEMIPD_ESHAPE, "local_attention: the matrix-core forms do not take this shape or type");
   if (form != 1 && mfma_ok) {
     const bool small = qk_dim <= 128 && v_dim <= 128;
     const int tile = 32 * v_tile_row_bytes(v_dim);                       // at most 32 * 576 bytes: below the 64 KB default
-    const bool sig = a.sigmoid != 0;
+    const bool sig = !POOL && a.sigmoid != 0;
     if (q_start == nullptr || max_q_len <= 1) {
       const int n_splits = (a.n_splits > 1 && a.partial != nullptr) ? a.n_splits : 1;
       a.n_splits = n_splits;
@@ -1248,10 +1468,10 @@ static int launch_local_attention(LocalAttnArgs a, int64_t max_q_len, int form, 
       int rc = -1;
 #define SEMIPD_LA_DEC(TT, NDD, NEE, NWW, SS, SLOT)                                                                              \
   do {                                                                                                                          \
-    if (lds > 65536 && ensure_dynamic_lds((const void*)local_attention_decode_kernel<TT, NDD, NEE, NWW, SS>, lds, done[SLOT],  \
+    if (lds > 65536 && ensure_dynamic_lds((const void*)local_attention_decode_kernel<TT, NDD, NEE, NWW, SS && !POOL, POOL>, kMaxDynLds, done[SLOT], \
                                           "local_attention"))                                                                   \
       return SEMIPD_EINVAL;                                                                                                     \
-    hipLaunchKernelGGL((local_attention_decode_kernel<TT, NDD, NEE, NWW, SS>), grid, dim3(64 * NWW), lds, as_stream(stream), a); \
+    hipLaunchKernelGGL((local_attention_decode_kernel<TT, NDD, NEE, NWW, SS && !POOL, POOL>), grid, dim3(64 * NWW), lds, as_stream(stream), a); \
     rc = 0;                                                                                                                     \
   } while (0)
       if (dtype == SEMIPD_BF16) {
@@ -1270,25 +1490,27 @@ static int launch_local_attention(LocalAttnArgs a, int64_t max_q_len, int form, 
       if (n_splits > 1) {
         const dim3 mgrid((unsigned)batch, (unsigned)num_q_heads);
         if (dtype == SEMIPD_BF16) {
-          if (sig) hipLaunchKernelGGL((local_attention_merge_kernel<bf16_t, true>), mgrid, dim3(64), 0, as_stream(stream), a);
-          else hipLaunchKernelGGL((local_attention_merge_kernel<bf16_t, false>), mgrid, dim3(64), 0, as_stream(stream), a);
+          if (sig) hipLaunchKernelGGL((local_attention_merge_kernel<bf16_t, !POOL, POOL>), mgrid, dim3(64), 0, as_stream(stream), a);
+          else hipLaunchKernelGGL((local_attention_merge_kernel<bf16_t, false, POOL>), mgrid, dim3(64), 0, as_stream(stream), a);
         } else {
-          if (sig) hipLaunchKernelGGL((local_attention_merge_kernel<f16_t, true>), mgrid, dim3(64), 0, as_stream(stream), a);
-          else hipLaunchKernelGGL((local_attention_merge_kernel<f16_t, false>), mgrid, dim3(64), 0, as_stream(stream), a);
+          if (sig) hipLaunchKernelGGL((local_attention_merge_kernel<f16_t, !POOL, POOL>), mgrid, dim3(64), 0, as_stream(stream), a);
+          else hipLaunchKernelGGL((local_attention_merge_kernel<f16_t, false, POOL>), mgrid, dim3(64), 0, as_stream(stream), a);
         }
       }
       return launch_status("local_attention_decode");
     }
     a.n_tiles = (num_tokens + 63) / 64 + batch;
     const dim3 grid((unsigned)((a.n_tiles * num_q_heads + 7) / 8 * 8));
-    const size_t tiles = 2 * ((size_t)tile + 32 * (size_t)(qk_dim * 2 + 32));   // two pairs of (32 V rows, 32 K rows): at most 71.7 KB
+    size_t tiles = 2 * ((size_t)tile + 32 * (size_t)(qk_dim * 2 + 32));   // two pairs of (32 V rows, 32 K rows): at most 71.7 KB
+    const size_t epilogue = 4 * 16 * (size_t)(v_dim + 4) * sizeof(float);       // POOL: the result in fp32
+    if (POOL && epilogue > tiles) tiles = epilogue;
     static std::atomic<uint64_t> done_p[8] = {};
 #define SEMIPD_LA_PRE(TT, NDD, NEE, SS, SLOT)                                                                                   \
   do {                                                                                                                          \
-    if (tiles > 65536 && ensure_dynamic_lds((const void*)local_attention_mfma_kernel<TT, NDD, NEE, SS>, tiles, done_p[SLOT],    \
+    if (tiles > 65536 && ensure_dynamic_lds((const void*)local_attention_mfma_kernel<TT, NDD, NEE, SS && !POOL, POOL>, kMaxDynLds, done_p[SLOT], \
                                             "local_attention"))                                                                 \
       return SEMIPD_EINVAL;                                                                                                     \
-    hipLaunchKernelGGL((local_attention_mfma_kernel<TT, NDD, NEE, SS>), grid, dim3(256), tiles, as_stream(stream), a);           \
+    hipLaunchKernelGGL((local_attention_mfma_kernel<TT, NDD, NEE, SS && !POOL, POOL>), grid, dim3(256), tiles, as_stream(stream), a);           \
   } while (0)
     if (dtype == SEMIPD_BF16) {
       if (small && !sig) SEMIPD_LA_PRE(bf16_t, 4, 8, false, 0);
@@ -1307,12 +1529,50 @@ static int launch_local_attention(LocalAttnArgs a, int64_t max_q_len, int form, 
   const dim3 grid((unsigned)((num_tokens + 3) / 4), (unsigned)num_q_heads);
   if (qk_dim <= 512 && v_dim <= 512) {
     SEMIPD_DISPATCH_DTYPE(dtype, T,
-                          hipLaunchKernelGGL((local_attention_rows_kernel<T, 8>), grid, dim3(256), 0, as_stream(stream), a));
+                          hipLaunchKernelGGL((local_attention_rows_kernel<T, 8, POOL>), grid, dim3(256), 0, as_stream(stream), a));
   } else {
     SEMIPD_DISPATCH_DTYPE(dtype, T,
-                          hipLaunchKernelGGL((local_attention_rows_kernel<T, 16>), grid, dim3(256), 0, as_stream(stream), a));
+                          hipLaunchKernelGGL((local_attention_rows_kernel<T, 16, POOL>), grid, dim3(256), 0, as_stream(stream), a));
   }
   return launch_status("local_attention");
+}
+
+static int launch_local_attention(LocalAttnArgs a, int64_t max_q_len, int form, int dtype, void* stream) {
+  return launch_attention<false>(a, max_q_len, form, dtype, stream);
+}
+
+// A sliding window whose far side is seen through block means (csrc/local_attention.hip: LocalAttnArgs::pool), softmax with a
+// sink term, the result turned back by the query's own angles and one gate per head.
+extern "C" int semipd_pooled_window_attention(const void* q, int64_t q_ld, const void* gate, int64_t gate_ld, void* out,
+                                              int64_t out_ld, const void* k_pool, const void* v_pool, const void* k_means,
+                                              const void* v_means, int k_piece, int v_piece, const int32_t* req_to_token,
+                                              int64_t req_to_token_stride, const int64_t* req_pool_indices,
+                                              const int64_t* seq_lens, const int32_t* q_start, const int32_t* q_len,
+                                              int64_t batch, int64_t num_tokens, int64_t max_q_len, int num_q_heads,
+                                              int num_kv_heads, int qk_dim, int v_dim, float scale, int window, int pool,
+                                              const float* sink, const float* turn, int n_splits, float* partial, int form,
+                                              int dtype, void* stream) {
+  SEMIPD_CHECK_ARG(window >= 0 && pool >= 0 && (pool == 0 || window > 0), SEMIPD_EINVAL,
+                   "pooled_window_attention: bad window or block size (blocks need a window)");
+  SEMIPD_CHECK_ARG(v_dim % 2 == 0, SEMIPD_ESHAPE, "pooled_window_attention: value heads of %d elements (pairs)", v_dim);
+  SEMIPD_CHECK_ARG(n_splits >= 0 && n_splits <= 64 && (n_splits <= 1 || partial != nullptr), SEMIPD_EINVAL,
+                   "pooled_window_attention: up to 64 slices of the keys, with room for their partial sums");
+  int k_sh = 0, v_sh = 0;
+  if (pool > 0) {
+    SEMIPD_CHECK_ARG(k_means && v_means, SEMIPD_EINVAL, "pooled_window_attention: blocks without their means");
+    while ((1 << k_sh) < k_piece) ++k_sh;
+    while ((1 << v_sh) < v_piece) ++v_sh;
+    const int unit = dtype == SEMIPD_F32 ? 4 : 8;
+    SEMIPD_CHECK_ARG((1 << k_sh) == k_piece && (1 << v_sh) == v_piece && k_piece >= unit && v_piece >= unit &&
+                         (int64_t)k_piece * pool >= qk_dim && (int64_t)v_piece * pool >= v_dim,
+                     SEMIPD_ESHAPE, "pooled_window_attention: pieces of %d / %d elements (powers of two that cover %d / %d in %d tokens)",
+                     k_piece, v_piece, qk_dim, v_dim, pool);
+  }
+  LocalAttnArgs a{q, q_ld, gate, gate_ld, out, out_ld, k_pool, v_pool, req_to_token, req_to_token_stride, req_pool_indices,
+                  seq_lens, q_start, q_len, batch, num_tokens, num_q_heads, num_kv_heads, qk_dim, v_dim, sink, scale, 0.f,
+                  0, 0, window, 0, nullptr, 0, 1.0f, 0, 0, n_splits, partial, 0, pool, k_means, v_means,
+                  (int64_t)num_kv_heads << k_sh, (int64_t)num_kv_heads << v_sh, k_sh, v_sh, turn};
+  return launch_attention<true>(a, max_q_len, form, dtype, stream);
 }
 
 extern "C" int semipd_latent_prep(const void* proj, int64_t ld, int64_t num_tokens, int num_heads, int dim, int rot_dim, int rank,

@@ -50,4 +50,15 @@ template <> __device__ inline uint32_t pack2<f16_t>(float a, float b) {
   return __builtin_bit_cast(uint32_t, __builtin_convertvector(v, f16x2_t));
 }
 
+// v_mfma_f32_16x16x32 (lane l: r = l & 15, g = l >> 4): a = A[row r][k 8g .. 8g+7], b = B[k 8g .. 8g+7][col r], d[i] = D[row 4g + i][col r]
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+template <typename T> __device__ __forceinline__ f32x4 mma16(const Frag16& a, const Frag16& b, f32x4 c);
+template <> __device__ __forceinline__ f32x4 mma16<bf16_t>(const Frag16& a, const Frag16& b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.b, b.b, c, 0, 0, 0);
+}
+template <> __device__ __forceinline__ f32x4 mma16<f16_t>(const Frag16& a, const Frag16& b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_f16(a.f, b.f, c, 0, 0, 0);
+}
+
 }  // namespace semipd

@@ -365,6 +365,41 @@ class HipAttnBackend(AttentionBackend):
             kt.stop("decode_attention" if forward_batch.forward_mode.is_decode() else "extend_attention", t0, 0.0, 0.0)
         return o
 
+    # ---- sliding window whose far side is seen through block means ---------------------------------------------------------
+    def forward_pooled_window(self, q, layer, forward_batch: ForwardBatch, sink=None, gate=None, turn=None):
+        """Softmax attention (+ sink) for layers whose descriptor carries `window` and `pool`, keys, values and block means
+        already in the pools (the layer named by layer_id may be another one than the caller's: its descriptor then carries
+        its own window and block size over that layer's rows).  The result is turned back by the rows of `turn` and
+        multiplied by sigmoid(gate [T, heads]).  One call for prompt portions, single tokens and decode batches."""
+        T = q.shape[0]
+        o = torch.empty((T, layer.tp_q_head_num * layer.v_head_dim), dtype=q.dtype, device=q.device)
+        pool = forward_batch.token_to_kv_pool
+        n_splits = 1
+        if forward_batch.forward_mode.is_decode():
+            q_start = q_len = None
+            max_q = 1
+            # (requests x key/value heads x groups of 16 heads) workgroups: below two per CU the keys of a request -- its
+            # window and the blocks in front of it -- are shared out over several, about 128 keys each at least
+            wgs = T * layer.tp_k_head_num * ((layer.tp_q_head_num // layer.tp_k_head_num + 15) // 16)
+            keys = self._decode_len_bound
+            if layer.window:
+                keys = min(keys, layer.window) + (max(0, keys - layer.window) // layer.pool if layer.pool else 0)
+            n_splits = max(1, min(16, (2 * max(1, self.num_cus)) // max(wgs, 1), keys // 128))
+            n_splits = int(os.environ.get("SEMIPD_POOLED_DECODE_SPLITS", n_splits))
+        else:
+            q_start, q_len = forward_batch.extend_start_loc, forward_batch.extend_seq_lens
+            max_q = max(forward_batch.extend_seq_lens_cpu)
+        kt = self._timing()
+        t0 = kt.start() if kt else None
+        ops.pooled_window_attention_fwd(q, o, pool.get_key_buffer(layer.layer_id), pool.get_value_buffer(layer.layer_id),
+                                        pool.get_block_means(layer.layer_id, layer.pool), self.req_to_token,
+                                        forward_batch.req_pool_indices, forward_batch.seq_lens, q_start, q_len, max_q, layer.scaling,
+                                        layer.window, sink=sink, gate=gate, turn=turn,
+                                        form=int(os.environ.get("SEMIPD_LOCAL_ATTN_FORM", "0")), n_splits=n_splits)
+        if kt:
+            kt.stop("decode_attention" if forward_batch.forward_mode.is_decode() else "extend_attention", t0, 0.0, 0.0)
+        return o
+
     # ---- decode: RoPE + KV store + attention + split merge in one launch -------------------------
     def fused_decode_waves(self, bs: int, head_dim: int, num_kv_splits: int = 0) -> int:
         """How a decode batch of `bs` requests goes from the qkv GEMM's planes to o_proj's input: 0 = the separate
@@ -431,7 +466,7 @@ class RadixAttention:
 
     def __init__(self, num_heads: int, head_dim: int, scaling: float, num_kv_heads: int, layer_id: int,
                  logit_cap: float = 0.0, v_head_dim: int = -1, chunk_size: int = 0, window: int = 0, keep_first: int = 0,
-                 sigmoid_weights: bool = False):
+                 sigmoid_weights: bool = False, pool: int = 0):
         self.tp_q_head_num = num_heads
         self.tp_k_head_num = num_kv_heads
         self.tp_v_head_num = num_kv_heads
@@ -447,6 +482,9 @@ class RadixAttention:
         # sliding window (HipAttnBackend.forward_window): the last `window` positions up to the query (0: all) plus the first
         # `keep_first` positions of the sequence; sigmoid_weights: independent sigmoid weights instead of a softmax
         self.window, self.keep_first, self.sigmoid_weights = int(window), int(keep_first), bool(sigmoid_weights)
+        # pooled window (HipAttnBackend.forward_pooled_window): the blocks of `pool` positions in front of the window are seen
+        # through their means (0: what has left the window is not seen at all)
+        self.pool = int(pool)
 
     def forward(self, q, k, v, forward_batch: ForwardBatch, save_kv_cache: bool = True):
         return forward_batch.attn_backend.forward(q, k, v, self, forward_batch, save_kv_cache)

@@ -129,6 +129,24 @@ class StreamRMSNorm(nn.Module):
         return ops.rms_stream(y, stream, next_norm.weight, next_norm.eps, next_norm.weight_shift)
 
 
+class OutputRMSNorm(nn.Module):
+    """RMS norm of a sublayer's OUTPUT in front of the sum on an fp32 residual stream (csrc/layernorm.hip: semipd_outnorm_stream;
+    fp32 arithmetic whatever the activation type): stream += y / sqrt(mean(y^2) + eps) * (weight + weight_shift); the sublayers
+    read the stream as it is.  `seam` also returns what comes next in the activation type: the new stream, or with a
+    StreamRMSNorm that norm of it (the one in front of the vocabulary head), from the same launch."""
+
+    def __init__(self, hidden_size: int, eps: float, weight_shift: float = 0.0, dtype=None):
+        super().__init__()
+        self.weight = nn.Parameter(torch.zeros(hidden_size, dtype=dtype) + (1.0 - weight_shift), requires_grad=False)
+        self.eps, self.weight_shift = float(eps), float(weight_shift)
+
+    def seam(self, y: torch.Tensor, stream: torch.Tensor, next_norm: Optional[StreamRMSNorm] = None) -> torch.Tensor:
+        if next_norm is None:
+            return ops.outnorm_stream(y, stream, self.weight, self.eps, self.weight_shift)
+        return ops.outnorm_stream(y, stream, self.weight, self.eps, self.weight_shift, next_weight=next_norm.weight,
+                                  next_eps=next_norm.eps, next_shift=next_norm.weight_shift)
+
+
 class BigramEmbedding(nn.Module):
     """Token embedding times a scale plus a row of a hashed table of token pairs, row (previous token * mul_prev + token *
     mul_cur) mod buckets, the table's last row for the first token of a sequence; the result is the start of an fp32 residual

@@ -161,6 +161,13 @@ def ipc_safe_zeros(shape, dtype: torch.dtype, device) -> torch.Tensor:
     return raw[:nbytes].view(dtype).view(*shape)
 
 
+def mean_piece(head_dim: int, block: int) -> int:
+    """Elements of a block mean that lie beside one token: the smallest power of two, 8 at least, that covers the head in
+    `block` tokens."""
+    need = max(8, -(-int(head_dim) // int(block)))
+    return 1 << (need - 1).bit_length()
+
+
 class MHATokenToKVPool:
     """K and V rows of every layer.  Layers of one geometry whose values are as wide as their keys share the slab
     kv[L, 2, N + page, Hkv, D] of the module docstring.  `head_num` / `head_dim` / `v_head_dim` may also be given per layer
@@ -168,11 +175,15 @@ class MHATokenToKVPool:
     after layer, keys [N + page, Hkv_l, D_l] in front of values [N + page, Hkv_l, Dv_l], each region starting on a
     256-byte boundary -- still one allocation and one IPC handle.  `values_in_keys`: a layer's values are the first
     v_head_dim elements of its key rows (latent attention: one row per token holds the latent and the shared rotated key
-    part, and the latent is the value); such a pool has no value regions, its value buffers are views of the key buffers."""
+    part, and the latent is the value); such a pool has no value regions, its value buffers are views of the key buffers.
+    `block_means`: per layer the block sizes (in tokens) whose mean key and mean value are kept next to the rows.  The mean of a
+    block is cut into pieces (`mean_piece` elements) and piece i lies at the slot of the block's token i, so the buffers are
+    [N + page, Hkv, piece] -- about 1 / block of the rows' memory -- and a block's mean is handed out and given back with its
+    tokens' slots."""
 
     def __init__(self, size: int, page_size: int, dtype: torch.dtype, head_num, head_dim,
                  layer_num: int, device: str, bypass_create_buffers: bool = False, v_head_dim=None,
-                 values_in_keys: bool = False):
+                 values_in_keys: bool = False, block_means=None):
         assert page_size == 1, "Semi-PD runs with token-granular pages (schedule_batch.py:937)"
         self.size, self.page_size, self.dtype = size, page_size, dtype
         self.layer_num, self.device = layer_num, device
@@ -192,6 +203,12 @@ class MHATokenToKVPool:
             raise ValueError("values_in_keys: one key/value head per layer whose values are a prefix of its key rows")
         self.uniform = (len(set(self.head_nums)) == 1 and len(set(self.head_dims)) == 1
                         and self.v_head_dims == self.head_dims and not self.values_in_keys)
+        self.block_sizes = [sorted(set(int(p) for p in s)) for s in block_means] if block_means else [[] for _ in range(layer_num)]
+        assert len(self.block_sizes) == layer_num
+        if any(self.block_sizes):
+            self.uniform = False
+        # per layer {block size: (key means, value means)}
+        self.means: List[dict] = [{} for _ in range(layer_num)]
         self.head_num, self.head_dim = self.head_nums[0], self.head_dims[0]
         self.k_buffer: List[torch.Tensor] = []
         self.v_buffer: List[torch.Tensor] = []
@@ -211,6 +228,12 @@ class MHATokenToKVPool:
             out.append((k_off, v_off))
         return out, off
 
+    def mean_shapes(self, layer_id: int):
+        """[(block size, shape of the key means, shape of the value means)] of a layer."""
+        rows, h = self.size + self.page_size, self.head_nums[layer_id]
+        return [(p, (rows, h, mean_piece(self.head_dims[layer_id], p)), (rows, h, mean_piece(self.v_head_dims[layer_id], p)))
+                for p in self.block_sizes[layer_id]]
+
     def _create_buffers(self):
         if self.uniform:
             # [L, 2, N+page, Hkv, D]: one allocation, one IPC handle
@@ -220,8 +243,17 @@ class MHATokenToKVPool:
             self.v_buffer = [self.slab[i, 1] for i in range(self.layer_num)]
             return
         regions, total = self._regions()
-        self.slab = ipc_safe_zeros((total,), torch.uint8, self.device)
         rows, es = self.size + self.page_size, self.dtype.itemsize
+        mean_at, off = [], total                     # block means behind all rows, every buffer on a 256-byte boundary
+        for i in range(self.layer_num):
+            for p, ks, vs in self.mean_shapes(i):
+                for kind, shape in ((0, ks), (1, vs)):
+                    mean_at.append((i, p, kind, shape, off))
+                    off = -(-(off + shape[0] * shape[1] * shape[2] * es) // 256) * 256
+        self.slab = ipc_safe_zeros((off,), torch.uint8, self.device)
+        for i, p, kind, shape, at in mean_at:
+            buf = self.slab[at: at + shape[0] * shape[1] * shape[2] * es].view(self.dtype).view(*shape)
+            self.means[i][p] = (buf,) if kind == 0 else self.means[i][p] + (buf,)
         for (k_off, v_off), h, d, dv, in_keys in zip(regions, self.head_nums, self.head_dims, self.v_head_dims, self.in_keys):
             self.k_buffer.append(self.slab[k_off: k_off + rows * h * d * es].view(self.dtype).view(rows, h, d))
             self.v_buffer.append(None if in_keys
@@ -239,7 +271,15 @@ class MHATokenToKVPool:
         rows, es = self.size + self.page_size, self.dtype.itemsize
         k = sum(rows * h * d * es for h, d in zip(self.head_nums, self.head_dims))
         v = sum(0 if f else rows * h * d * es for h, d, f in zip(self.head_nums, self.v_head_dims, self.in_keys))
+        for i in range(self.layer_num):
+            for _, ks, vs in self.mean_shapes(i):
+                k += ks[0] * ks[1] * ks[2] * es
+                v += vs[0] * vs[1] * vs[2] * es
         return k, v
+
+    def get_block_means(self, layer_id: int, block: int):
+        """(block, key means, value means) of a layer; None for block 0."""
+        return (block, *self.means[layer_id][block]) if block else None
 
     def get_key_buffer(self, layer_id: int):
         return self.k_buffer[layer_id]

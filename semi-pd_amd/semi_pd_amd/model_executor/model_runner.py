@@ -26,7 +26,7 @@ from semi_pd_amd.distributed import (get_tensor_model_parallel_rank, get_tensor_
 from semi_pd_amd.layers.attention_backend import HipAttnBackend
 from semi_pd_amd.layers.basic import Sampler
 from semi_pd_amd.mem_cache.memory_pool import (MHATokenToKVPool, MLATokenToKVPool, RecurrentStatePool, ReqToTokenPool,
-                                               TokenToKVPoolAllocator)
+                                               TokenToKVPoolAllocator, mean_piece)
 from semi_pd_amd.model_executor.forward_batch_info import ForwardBatch, ForwardMode
 from semi_pd_amd.semi_pd.utils import (InstanceRole, IPCInfo, convert_ipc_handle_to_tensor, get_device_sm_count,
                                        get_ipc_handle)
@@ -57,6 +57,9 @@ def build_model(model_config, dtype):
     if arch == "Tibenex":
         from semi_pd_amd.models.tibenex import TibenexForCausalLM
         return TibenexForCausalLM(model_config, dtype)
+    if arch == "Gukidra":
+        from semi_pd_amd.models.gukidra import GukidraForCausalLM
+        return GukidraForCausalLM(model_config, dtype)
     raise ValueError(f"unsupported architecture {arch}")
 
 
@@ -300,8 +303,10 @@ class ModelRunner:
             if not isinstance(in_keys, (list, tuple)):
                 in_keys = [bool(in_keys)] * len(geo["num_kv_heads"])
             cell = sum(h * (d + (0 if f else dv))
-                       for h, d, dv, f in zip(geo["num_kv_heads"], geo["head_dim"], geo["v_head_dim"], in_keys)) \
-                * self.kv_cache_dtype.itemsize
+                       for h, d, dv, f in zip(geo["num_kv_heads"], geo["head_dim"], geo["v_head_dim"], in_keys))
+            for h, d, dv, blocks in zip(geo["num_kv_heads"], geo["head_dim"], geo["v_head_dim"], geo.get("block_means") or ()):
+                cell += sum(h * (mean_piece(d, p) + mean_piece(dv, p)) for p in set(blocks))
+            cell *= self.kv_cache_dtype.itemsize
         else:
             cell = (geo["num_kv_heads"] * (geo["head_dim"] + geo["v_head_dim"]) * geo["num_layers"]
                     * self.kv_cache_dtype.itemsize)
@@ -333,7 +338,8 @@ class ModelRunner:
             self.token_to_kv_pool = MHATokenToKVPool(self.max_total_num_tokens, 1, self.kv_cache_dtype,
                                                      geo["num_kv_heads"], geo["head_dim"], geo["num_layers"],
                                                      dev, bypass_create_buffers=bypass, v_head_dim=geo["v_head_dim"],
-                                                     values_in_keys=geo.get("values_in_keys") or False)
+                                                     values_in_keys=geo.get("values_in_keys") or False,
+                                                     block_means=geo.get("block_means"))
         self.token_to_kv_pool_allocator = TokenToKVPoolAllocator(self.max_total_num_tokens, self.kv_cache_dtype, dev,
                                                                  self.token_to_kv_pool)
         # models with recurrent layers: one fp32 state row per running request (`state_geometry`: the width of every
@@ -391,7 +397,8 @@ class ModelRunner:
             for i in range(pool.layer_num):
                 # (values that are views of the key rows travel with the keys' handle)
                 kv_handles.append([get_ipc_handle(pool.k_buffer[i]),
-                                   None if pool.in_keys[i] else get_ipc_handle(pool.v_buffer[i])])
+                                   None if pool.in_keys[i] else get_ipc_handle(pool.v_buffer[i])]
+                                  + [get_ipc_handle(m) for p in pool.block_sizes[i] for m in pool.means[i][p]])
             kv_info = {"kind": "mha", "shape": tuple(pool.k_buffer[0].shape), "dtype": pool.dtype,
                        "numel": pool.k_buffer[0].numel(), "layer_num": pool.layer_num}
             if not pool.uniform:
@@ -467,6 +474,9 @@ class ModelRunner:
             pool.v_buffer = [None if h[1] is None else one(h[1], sh[1]) for h, sh in zip(ipc_info.kv_cache_handles, kvi["shapes"])]
             if pool.values_in_keys:
                 pool.link_value_views()
+            for i, handles in enumerate(ipc_info.kv_cache_handles):       # behind keys and values: the block means, by block size
+                for n, (p, ks, vs) in enumerate(pool.mean_shapes(i)):
+                    pool.means[i][p] = (one(handles[2 + 2 * n], ks), one(handles[3 + 2 * n], vs))
         elif kvi["kind"] == "mha":
             pool.k_buffer = [self._import(h[0], info) for h in ipc_info.kv_cache_handles]
             pool.v_buffer = [self._import(h[1], info) for h in ipc_info.kv_cache_handles]

@@ -25,12 +25,13 @@ from torch import nn
 def _config_classes():
     from semi_pd_amd.models.deepseek_v2 import DeepseekV2Config
     from semi_pd_amd.models.llama import LlamaConfig
+    from semi_pd_amd.models.gukidra import GukidraConfig
     from semi_pd_amd.models.kudirax import KudiraxConfig
     from semi_pd_amd.models.opt import OPTConfig
     from semi_pd_amd.models.penozen import PenozenConfig
     from semi_pd_amd.models.tibenex import TibenexConfig
     from semi_pd_amd.models.tigotar import TigotarConfig
-    return {"Tibenex": TibenexConfig, "Tigotar": TigotarConfig, "Penozen": PenozenConfig, "LlamaForCausalLM": LlamaConfig, "OPTForCausalLM": OPTConfig,
+    return {"Gukidra": GukidraConfig, "Tibenex": TibenexConfig, "Tigotar": TigotarConfig, "Penozen": PenozenConfig, "LlamaForCausalLM": LlamaConfig, "OPTForCausalLM": OPTConfig,
             "DeepseekV2ForCausalLM": DeepseekV2Config, "DeepseekV3ForCausalLM": DeepseekV2Config,
             "Kudirax": KudiraxConfig}
 
@@ -352,6 +353,66 @@ def _tibenex_items(config, weights):
         raise RuntimeError(f"checkpoint ended with incomplete stacked parameters: {list(st.pending)[:4]}")
 
 
+_GUKIDRA_RE = re.compile(r"^l(\d+)\.(mix|mlp|norm1|norm2)(?:\.(.+))?$")
+_GUKIDRA_ATTN_IN = ("q", "k", "v", "g")
+_GUKIDRA_SHARED_IN = ("q", "g")                 # a layer that reads another layer's keys and values
+_GUKIDRA_MEMORY_IN = ("q", "k", "v", "g", "i", "f")
+_GUKIDRA_ATTN_LEAF = {"q.norm": "q_norm", "k.norm": "k_norm", "o": "out_proj.weight"}
+_GUKIDRA_MEMORY_LEAF = {"norm": "out_norm", "i.b": "i_bias", "f.b": "f_bias", "o": "out_proj.weight"}
+
+
+def _gukidra_items(config, weights):
+    """Gukidra checkpoint names (embed, l<i>.norm1|norm2, l<i>.mix.q|q.norm|k|k.norm|v|g|o of an attention layer -- without k, k.norm
+    and v where it reads another layer's cache --, l<i>.mix.q|k|v|g|o|norm|i|i.b|f|f.b of a matrix-memory layer,
+    l<i>.mlp.gate|up|down, final.norm) -> product parameters: q | k | v | g (| i | f) stack into the mixer's merged input
+    projection, followed by the zero rows that bring it to a multiple of 8; gate and up into the feed-forward's."""
+    st = _Stacker()
+    top = {"embed": "embed.weight", "final.norm": "final_norm.weight"}
+    for name, t in weights:
+        if name in top:
+            yield top[name], t
+            continue
+        m = _GUKIDRA_RE.match(name)
+        if not m or int(m.group(1)) >= len(config.layers):
+            raise KeyError(f"checkpoint tensor {name} has no counterpart in a Gukidra model")
+        i, part, leaf = int(m.group(1)), m.group(2), m.group(3)
+        base = f"layers.{i}."
+        lc = config.layers[i]
+        if part in ("norm1", "norm2"):
+            if leaf is not None:
+                raise KeyError(f"checkpoint tensor {name} has no counterpart in a Gukidra model")
+            if part == "norm2" and not lc.ff:
+                continue                      # a layer without feed-forward has no second output to norm
+            yield base + part + ".weight", t
+        elif part == "mix":
+            if lc.kind == "attention":
+                shared = lc.mixer.kv_from is not None
+                parts, leaves = (_GUKIDRA_SHARED_IN if shared else _GUKIDRA_ATTN_IN), _GUKIDRA_ATTN_LEAF
+                if shared and leaf in ("k", "k.norm", "v"):
+                    raise KeyError(f"checkpoint tensor {name}: layer {i} reads the keys and values of layer {lc.mixer.kv_from}")
+            else:
+                parts, leaves = _GUKIDRA_MEMORY_IN, _GUKIDRA_MEMORY_LEAF
+            if leaf in parts:
+                for done_name, full in st.add(base + "mix.in_proj.weight", parts.index(leaf), len(parts), t):
+                    pad = -full.shape[0] % 8
+                    yield done_name, torch.cat([full, full.new_zeros(pad, full.shape[1])], 0) if pad else full
+            elif leaf in leaves:
+                yield base + "mix." + leaves[leaf], t
+            else:
+                raise KeyError(f"checkpoint tensor {name} has no counterpart in a layer of type {lc.kind}")
+        else:
+            if not lc.ff:
+                raise KeyError(f"checkpoint tensor {name}: layer {i} has no feed-forward")
+            if leaf in ("gate", "up"):
+                yield from st.add(base + "mlp.gate_up_proj.weight", int(leaf == "up"), 2, t)
+            elif leaf == "down":
+                yield base + "mlp.down_proj.weight", t
+            else:
+                raise KeyError(f"checkpoint tensor {name} has no counterpart in a Gukidra model")
+    if st.pending:
+        raise RuntimeError(f"checkpoint ended with incomplete stacked parameters: {list(st.pending)[:4]}")
+
+
 _EXPERT_RE = re.compile(r"^(.*\.mlp\.experts)\.(\d+)\.(gate_proj|up_proj|down_proj)\.(weight|weight_scale_inv)$")
 
 
@@ -369,6 +430,9 @@ def product_items(config, weights: Iterable[Tuple[str, torch.Tensor]]) -> Iterat
         return
     if arch == "Tibenex":
         yield from _tibenex_items(config, weights)
+        return
+    if arch == "Gukidra":
+        yield from _gukidra_items(config, weights)
         return
     st = _Stacker()
     tie = bool(getattr(config, "tie_word_embeddings", False))

@@ -1813,14 +1813,16 @@ def sigmoid_gate_heads_(x: torch.Tensor, gate: torch.Tensor) -> torch.Tensor:
     return x
 
 
-def embed_stream(input_ids: torch.Tensor, embed: torch.Tensor, scale: float) -> torch.Tensor:
-    """fp32 [T, width] = embed[id] * scale: the start of an fp32 residual stream (csrc/layernorm.hip)."""
+def embed_stream(input_ids: torch.Tensor, embed: torch.Tensor, scale: float, want_copy: bool = False):
+    """fp32 [T, width] = embed[id] * scale: the start of an fp32 residual stream (csrc/layernorm.hip); want_copy: (stream, the
+    same rows in the embedding's type)."""
     if input_ids.dtype != torch.int64 or not input_ids.is_contiguous() or embed.dim() != 2 or not embed.is_contiguous():
         raise RuntimeError("embed_stream: int64 ids, embed [V, W] contiguous")
     out = torch.empty((input_ids.shape[0], embed.shape[1]), dtype=torch.float32, device=embed.device)
-    check(_lib.load().semipd_embed_stream(ptr(input_ids), ptr(embed), float(scale), input_ids.shape[0], ptr(out), embed.shape[1],
-                                          dtype_code(embed.dtype), current_stream(embed.device)), "embed_stream")
-    return out
+    copy = torch.empty_like(out, dtype=embed.dtype) if want_copy else None
+    check(_lib.load().semipd_embed_stream(ptr(input_ids), ptr(embed), float(scale), input_ids.shape[0], ptr(out), ptr(copy),
+                                          embed.shape[1], dtype_code(embed.dtype), current_stream(embed.device)), "embed_stream")
+    return (out, copy) if want_copy else out
 
 
 def postnorm_stream(y: Optional[torch.Tensor], layer_scale: Optional[torch.Tensor], stream: torch.Tensor, alpha: float,
@@ -2018,4 +2020,197 @@ def state_space(proj: torch.Tensor, z_off: int, x_off: int, dt_off: int, conv_w:
                                  ptr(state_indices), ptr(seq_lens), ptr(q_start), ptr(q_len), B, T, num_heads, groups, state_size,
                                  v_dim, taps, ptr(out), out.stride(0), 1 if fused else 0, dtype_code(proj.dtype),
                                  current_stream(proj.device)), "state_space")
+    return out
+
+
+# ---- norm of a sublayer's output, pooled window attention with turned values, matrix memory -------------------------------
+def outnorm_stream(y: torch.Tensor, stream: torch.Tensor, weight: torch.Tensor, eps: float, weight_shift: float = 0.0,
+                   want_out: bool = True, next_weight: Optional[torch.Tensor] = None, next_eps: float = 0.0,
+                   next_shift: float = 0.0) -> Optional[torch.Tensor]:
+    """stream (fp32 [rows, width], in place) += y / sqrt(mean(y^2) + eps) * (weight + weight_shift).  Returns (None with
+    want_out=False) the new stream in y's type, or with next_weight its own RMS norm times (next_weight + next_shift)
+    (csrc/layernorm.hip: semipd_outnorm_stream)."""
+    if stream.dim() != 2 or stream.dtype != torch.float32 or stream.stride(1) != 1:
+        raise RuntimeError("outnorm_stream: the stream is fp32 [rows, width] with contiguous rows")
+    rows, width = stream.shape
+    if y.shape != stream.shape or y.stride(1) != 1:
+        raise RuntimeError("outnorm_stream: y is shaped like the stream, with contiguous rows")
+    for w in (weight, next_weight):
+        if w is not None and (w.shape != (width,) or w.dtype != y.dtype or not w.is_contiguous()):
+            raise RuntimeError("outnorm_stream: weights are contiguous [width] of y's type")
+    if next_weight is not None and not want_out:
+        raise RuntimeError("outnorm_stream: a second norm without an output")
+    out = torch.empty((rows, width), dtype=y.dtype, device=y.device) if want_out else None
+    check(_lib.load().semipd_outnorm_stream(ptr(y), y.stride(0), ptr(stream), stream.stride(0), ptr(weight), float(weight_shift),
+                                            float(eps), ptr(next_weight), float(next_shift), float(next_eps), ptr(out),
+                                            out.stride(0) if out is not None else 0, rows, width, dtype_code(y.dtype),
+                                            current_stream(y.device)), "outnorm_stream")
+    return out
+
+
+def angle_table(positions: torch.Tensor, freq: torch.Tensor) -> torch.Tensor:
+    """fp32 [T, len(freq), 2]: cos and sin of position * freq (csrc/attention_prep.hip)."""
+    if positions.dtype != torch.int64 or not positions.is_contiguous() or freq.dtype != torch.float32 or not freq.is_contiguous():
+        raise RuntimeError("angle_table: int64 positions, fp32 frequencies")
+    T, half = positions.shape[0], freq.numel()
+    out = torch.empty((T, half, 2), dtype=torch.float32, device=positions.device)
+    check(_lib.load().semipd_angle_table(ptr(positions), ptr(freq), half, T, ptr(out), current_stream(positions.device)), "angle_table")
+    return out
+
+
+def _check_angles(name: str, table: Optional[torch.Tensor], T: int, half: int) -> None:
+    if table is not None and (table.dtype != torch.float32 or table.shape != (T, half, 2) or not table.is_contiguous()):
+        raise RuntimeError(f"{name}: angle tables are contiguous fp32 [{T}, {half}, 2]")
+
+
+def _check_means(name: str, means, k_buffer: torch.Tensor, v_buffer: torch.Tensor) -> None:
+    """means: (tokens of a block, key means [N, G, piece], value means [N, G, piece]) or None."""
+    if means is None:
+        return
+    pool, km, vm = means
+    for m, buf in ((km, k_buffer), (vm, v_buffer)):
+        if m.dim() != 3 or m.shape[:2] != buf.shape[:2] or m.dtype != buf.dtype or not m.is_contiguous() \
+                or m.shape[2] * pool < buf.shape[2]:
+            raise RuntimeError(f"{name}: block means are contiguous [N, G, piece] buffers next to the pools, piece * block >= head size")
+
+
+def head_norm_rope_kv_store(qkv: torch.Tensor, num_q_heads: int, num_kv_heads: int, qk_dim: int, v_dim: int, k_off: int, v_off: int,
+                            q_weight: torch.Tensor, k_weight: Optional[torch.Tensor], eps: float, qk_angles: Optional[torch.Tensor],
+                            rot_dims: int, v_angles: Optional[torch.Tensor], k_buffer: Optional[torch.Tensor],
+                            v_buffer: Optional[torch.Tensor], loc: Optional[torch.Tensor], means=None,
+                            positions: Optional[torch.Tensor] = None, req_to_token: Optional[torch.Tensor] = None,
+                            req_pool_indices: Optional[torch.Tensor] = None, seq_lens: Optional[torch.Tensor] = None,
+                            q_start: Optional[torch.Tensor] = None, q_len: Optional[torch.Tensor] = None) -> None:
+    """Rows of `qkv` hold q | k | v at columns 0, k_off, v_off (num_kv_heads = 0: queries only).  Every q / k head to unit RMS times
+    a weight [qk_dim], its first rot_dims elements turned in pairs (i, i + rot_dims / 2) by qk_angles; every v head turned in
+    pairs (m, m + v_dim / 2) by v_angles; q in place, k / v into the pools at `loc`.  `means` = (block size, key means, value
+    means): the blocks that the batch completes get their means as well (csrc/attention_prep.hip)."""
+    name = "head_norm_rope_kv_store"
+    if qkv.dim() != 2 or qkv.stride(1) != 1:
+        raise RuntimeError(f"{name}: qkv must be 2-D with contiguous rows")
+    T = qkv.shape[0]
+    for w_ in (q_weight, k_weight):
+        if w_ is not None and (w_.shape != (qk_dim,) or w_.dtype != qkv.dtype or not w_.is_contiguous()):
+            raise RuntimeError(f"{name}: norm weights are contiguous [{qk_dim}] of the activation type")
+    if rot_dims:
+        _check_angles(name, qk_angles, T, rot_dims // 2)
+    B = 0
+    if num_kv_heads:
+        _check_angles(name, v_angles, T, v_dim // 2)
+        if loc.dtype != torch.int64 or loc.shape[0] != T:
+            raise RuntimeError(f"{name}: one int64 pool slot per row")
+        for buf, size in ((k_buffer, qk_dim), (v_buffer, v_dim)):
+            if buf.dtype != qkv.dtype or buf.dim() != 3 or buf.shape[1:] != (num_kv_heads, size) or not buf.is_contiguous():
+                raise RuntimeError(f"{name}: pools must be contiguous [N, {num_kv_heads}, size] of {qkv.dtype}")
+        if means is not None:
+            _check_means(name, means, k_buffer, v_buffer)
+            B = req_pool_indices.shape[0]
+            _batch_rows(name, T, B, q_start, q_len)
+            if req_to_token.dtype != torch.int32 or req_pool_indices.dtype != torch.int64 or seq_lens.dtype != torch.int64 \
+                    or positions.dtype != torch.int64 or positions.shape[0] != T:
+                raise RuntimeError(f"{name}: req_to_token int32, req_pool_indices / seq_lens / positions int64")
+    pool, km, vm = means if means is not None else (0, None, None)
+    check(_lib.load().semipd_head_norm_rope_kv_store(
+        ptr(qkv), qkv.stride(0), T, num_q_heads, num_kv_heads, qk_dim, v_dim, int(k_off), int(v_off), ptr(q_weight), ptr(k_weight),
+        float(eps), ptr(qk_angles) if rot_dims else None, int(rot_dims), ptr(v_angles), ptr(k_buffer), ptr(v_buffer), ptr(loc),
+        ptr(positions) if pool else None, int(pool), ptr(km), ptr(vm), km.shape[2] if pool else 0, vm.shape[2] if pool else 0,
+        ptr(req_to_token) if pool else None, req_to_token.stride(0) if pool else 0, ptr(req_pool_indices) if pool else None,
+        ptr(seq_lens) if pool else None, ptr(q_start) if pool else None, ptr(q_len) if pool else None, B, dtype_code(qkv.dtype),
+        current_stream(qkv.device)), name)
+
+
+def block_means(k_buffer: torch.Tensor, v_buffer: torch.Tensor, means, req_to_token: torch.Tensor, req_pool_indices: torch.Tensor,
+                seq_lens: torch.Tensor, q_start: Optional[torch.Tensor], q_len: Optional[torch.Tensor], num_tokens: int) -> None:
+    """The means of the blocks of means[0] tokens that the batch's rows complete, over what the pools hold
+    (csrc/attention_prep.hip: semipd_block_means)."""
+    _check_means("block_means", means, k_buffer, v_buffer)
+    pool, km, vm = means
+    B = req_pool_indices.shape[0]
+    _batch_rows("block_means", num_tokens, B, q_start, q_len)
+    if req_to_token.dtype != torch.int32 or req_pool_indices.dtype != torch.int64 or seq_lens.dtype != torch.int64:
+        raise RuntimeError("block_means: req_to_token int32, req_pool_indices / seq_lens int64")
+    check(_lib.load().semipd_block_means(ptr(k_buffer), ptr(v_buffer), k_buffer.shape[1], k_buffer.shape[2], v_buffer.shape[2], int(pool),
+                                         ptr(km), ptr(vm), km.shape[2], vm.shape[2], ptr(req_to_token), req_to_token.stride(0),
+                                         ptr(req_pool_indices), ptr(seq_lens), ptr(q_start), ptr(q_len), B, int(num_tokens),
+                                         dtype_code(k_buffer.dtype), current_stream(k_buffer.device)), "block_means")
+
+
+def pooled_window_attention_fwd(q: torch.Tensor, out: torch.Tensor, k_buffer: torch.Tensor, v_buffer: torch.Tensor, means,
+                                req_to_token: torch.Tensor, req_pool_indices: torch.Tensor, seq_lens: torch.Tensor,
+                                q_start: Optional[torch.Tensor], q_len: Optional[torch.Tensor], max_q_len: int, sm_scale: float,
+                                window: int, sink: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+                                turn: Optional[torch.Tensor] = None, form: int = 0, n_splits: int = 1) -> None:
+    """Softmax attention over the last `window` positions (0: all) and, in the same softmax, over the means of the blocks whose
+    last token is at least `window` back (means = (block size, key means, value means); None: no blocks).  sink fp32 [H]; the
+    result is turned back by `turn` (an angle table over v_dim / 2 pairs) and multiplied by sigmoid(gate [T, H]).  Batch
+    description as in local_attention_fwd (csrc/local_attention.hip: semipd_pooled_window_attention)."""
+    name = "pooled_window_attention_fwd"
+    T = q.shape[0]
+    G, D, E = k_buffer.shape[1], k_buffer.shape[2], v_buffer.shape[2]
+    if q.dim() != 2 or out.dim() != 2 or q.stride(1) != 1 or out.stride(1) != 1 or q.shape[1] % D:
+        raise RuntimeError(f"{name}: q / out are [T, heads * size] with contiguous rows")
+    H = q.shape[1] // D
+    if out.shape != (T, H * E) or out.dtype != q.dtype or k_buffer.dtype != q.dtype or v_buffer.dtype != q.dtype:
+        raise RuntimeError(f"{name}: shapes or types of q, out and the pools disagree")
+    if not (k_buffer.is_contiguous() and v_buffer.is_contiguous()) or v_buffer.shape[1] != G or H % G:
+        raise RuntimeError(f"{name}: pools must be contiguous [N, G, size], heads a multiple of G")
+    _check_means(name, means, k_buffer, v_buffer)
+    _check_angles(name, turn, T, E // 2)
+    if sink is not None and (sink.dtype != torch.float32 or sink.numel() != H or not sink.is_contiguous()):
+        raise RuntimeError(f"{name}: sink is fp32 [H]")
+    if gate is not None and (gate.shape != (T, H) or gate.dtype != q.dtype or gate.stride(1) != 1):
+        raise RuntimeError(f"{name}: gate is [T, H] of q's type")
+    if req_to_token.dtype != torch.int32 or req_pool_indices.dtype != torch.int64 or seq_lens.dtype != torch.int64:
+        raise RuntimeError(f"{name}: req_to_token int32, req_pool_indices / seq_lens int64")
+    B = req_pool_indices.shape[0]
+    _batch_rows(name, T, B, q_start, q_len)
+    n_splits = int(n_splits) if (q_start is None and q.dtype != torch.float32) else 1
+    partial = torch.empty((T, H, n_splits, E + 2), dtype=torch.float32, device=q.device) if n_splits > 1 else None
+    pool, km, vm = means if means is not None else (0, None, None)
+    check(_lib.load().semipd_pooled_window_attention(
+        ptr(q), q.stride(0), ptr(gate), gate.stride(0) if gate is not None else 0, ptr(out), out.stride(0), ptr(k_buffer), ptr(v_buffer),
+        ptr(km), ptr(vm), km.shape[2] if pool else 0, vm.shape[2] if pool else 0, ptr(req_to_token), req_to_token.stride(0),
+        ptr(req_pool_indices), ptr(seq_lens), ptr(q_start), ptr(q_len), B, T, int(max_q_len), H, G, D, E, float(sm_scale), int(window),
+        int(pool), ptr(sink), ptr(turn), n_splits, ptr(partial), int(form), dtype_code(q.dtype), current_stream(q.device)), name)
+
+
+def matrix_memory_state_width(num_heads: int, qk_dim: int, v_dim: int) -> int:
+    """fp32 elements of a request's state: S [H, D, E] | n [H, D] | m [H]."""
+    return num_heads * qk_dim * v_dim + num_heads * qk_dim + num_heads
+
+
+def matrix_memory(proj: torch.Tensor, offsets, num_heads: int, qk_dim: int, v_dim: int, i_bias: torch.Tensor, f_bias: torch.Tensor,
+                  gate_cap: float, norm_weight: torch.Tensor, eps: float, state: torch.Tensor, state_indices: torch.Tensor,
+                  seq_lens: torch.Tensor, q_start: Optional[torch.Tensor], q_len: Optional[torch.Tensor], form: int = 0) -> torch.Tensor:
+    """The matrix memory behind its projection GEMM (csrc/matrix_memory.hip).  offsets: columns of q, k, v, the output gate, the
+    input gates and the forget gates in the rows of `proj`; i_bias / f_bias fp32 [H]; norm_weight [H * E]; state fp32 [slots,
+    matrix_memory_state_width] is a column range of the requests' state rows.  Returns [T, H * E]."""
+    T, B = proj.shape[0], state_indices.shape[0]
+    inner = num_heads * v_dim
+    if proj.dim() != 2 or proj.stride(1) != 1:
+        raise RuntimeError("matrix_memory: proj is 2-D with contiguous rows")
+    q_off, k_off, v_off, g_off, i_off, f_off = (int(o) for o in offsets)
+    qk = num_heads * qk_dim
+    if min(offsets) < 0 or max(q_off + qk, k_off + qk, v_off + inner, g_off + inner, i_off + num_heads, f_off + num_heads) > proj.shape[1]:
+        raise RuntimeError("matrix_memory: a column range leaves the row")
+    for vec in (i_bias, f_bias):
+        if vec.dtype != torch.float32 or vec.shape != (num_heads,) or not vec.is_contiguous():
+            raise RuntimeError("matrix_memory: gate biases are fp32 [H]")
+    if norm_weight.shape != (inner,) or norm_weight.dtype != proj.dtype or not norm_weight.is_contiguous():
+        raise RuntimeError("matrix_memory: norm_weight is contiguous [H * E] of the activation type")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] != matrix_memory_state_width(num_heads, qk_dim, v_dim) \
+            or state.stride(1) != 1:
+        raise RuntimeError("matrix_memory: state is fp32 [slots, H * D * E + H * D + H]")
+    if state_indices.dtype != torch.int64 or seq_lens.dtype != torch.int64 or seq_lens.shape[0] != B:
+        raise RuntimeError("matrix_memory: state_indices / seq_lens are int64 [B]")
+    _batch_rows("matrix_memory", T, B, q_start, q_len)
+    lib = _lib.load()
+    wld = int(lib.semipd_matrix_memory_work_width(num_heads, v_dim))
+    work = torch.empty((T, wld), dtype=torch.float32, device=proj.device)
+    out = torch.empty((T, inner), dtype=proj.dtype, device=proj.device)
+    check(lib.semipd_matrix_memory(ptr(proj), proj.stride(0), q_off, k_off, v_off, g_off, i_off, f_off, ptr(i_bias), ptr(f_bias),
+                                   float(gate_cap), ptr(norm_weight), float(eps), ptr(work), wld, ptr(state), state.stride(0),
+                                   ptr(state_indices), ptr(seq_lens), ptr(q_start), ptr(q_len), B, T, num_heads, qk_dim, v_dim,
+                                   float(qk_dim) ** -0.5, ptr(out), out.stride(0), int(form), dtype_code(proj.dtype),
+                                   current_stream(proj.device)), "matrix_memory")
     return out
