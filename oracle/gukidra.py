@@ -200,7 +200,9 @@ def random_weights(cfg: dict, seed: int = 0) -> Dict[str, torch.Tensor]:
                 w[pre + "mix.v"] = mat(G * E, W)
                 w[pre + "mix.k.norm"] = vec(D, 0.2, 1.5)
         else:
-            w[pre + "mix.k"] = mat(H * D, W)
+            # (keys that lean towards the token's own query: a read-out of near-zero q . k keeps its direction only up to rounding
+            # once every head is brought to unit RMS, and the comparison would be one of signs)
+            w[pre + "mix.k"] = (0.8 * w[pre + "mix.q"].float() + 0.6 * mat(H * D, W).float()).to(torch.bfloat16)
             w[pre + "mix.v"] = mat(H * E, W)
             w[pre + "mix.g"] = mat(H * E, W)
             w[pre + "mix.norm"] = vec(H * E, 0.1, 1.0)

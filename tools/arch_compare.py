@@ -4,7 +4,9 @@ sublayers' outputs, attention over a bounded range of keys through the same kern
 with `--arch-design penozen`: Penozen next to Tigotar (fp32 stream, attention and a recurrence over pooled state rows,
 a mixture of experts behind them);
 with `--arch-design tibenex`: Tibenex next to Penozen (fp32 stream, latent attention, a recurrence with a matrix state and a
-short convolution over pooled state rows).
+short convolution over pooled state rows);
+with `--arch-design gukidra`: Gukidra next to Tibenex (fp32 stream with a norm behind every sublayer, attention and a recurrence
+with a matrix state over pooled state rows, a dense feed-forward), its windowed attention next to Tigotar's window kernel.
 
 Two parts, printed as one JSON object:
   * "models": prefill and decode throughput of a few-layer model of each design at layer sizes of real models, both driven
@@ -762,7 +764,168 @@ def main_tibenex(args) -> dict:
     return result
 
 
+GUKIDRA_SIZES = {
+    # name: hidden, ff, vocab, attention heads / kv heads / head size, window and block, memory heads / key size / value size (the
+    # state of a memory layer has as many elements as that of Tibenex's state-space layer)
+    "8b-layer": dict(hidden=4096, ff=14336, vocab=32000, heads=32, kv=8, dim=128, window=1024, pool=16, mheads=8, mdim=256, mvdim=512),
+    "3b-layer": dict(hidden=3072, ff=8192, vocab=32000, heads=24, kv=8, dim=128, window=1024, pool=16, mheads=6, mdim=256, mvdim=512),
+    "1b-layer": dict(hidden=2048, ff=8192, vocab=32000, heads=32, kv=8, dim=64, window=1024, pool=16, mheads=8, mdim=128, mvdim=256),
+}
+
+
+def _gukidra_kernel_pairs(s, tb, dev):
+    """[(what, Gukidra kernel's record, like kernel's record)]: `s` Gukidra's layer shape, `tb` Tibenex's at the same size."""
+    from semi_pd_amd import ops
+    from semi_pd_amd.mem_cache.memory_pool import mean_piece
+    dt = torch.bfloat16
+    W = s["hidden"]
+    out = []
+
+    def rec(tm, nbytes=0.0, flops=0.0, vflops=0.0):
+        frac = max(nbytes / tm / HBM, flops / tm / MFMA, vflops / tm / VALU)
+        return {"us": round(tm * 1e6, 1), "TB_per_s": round(nbytes / tm / 1e12, 2),
+                "TFLOP_per_s": round(max(flops, vflops) / tm / 1e12, 1), "of_roofline": round(frac, 3)}
+
+    B, L = 4, 2048
+    T = B * L
+    B2, C = 32, 2000
+    rows, lens = torch.arange(B, device=dev), torch.full((B,), L, device=dev, dtype=torch.int64)
+    q_start = torch.arange(B, device=dev, dtype=torch.int32) * L
+    q_len = torch.full((B,), L, device=dev, dtype=torch.int32)
+    rows2, lens2 = torch.arange(B2, device=dev), torch.full((B2,), C, device=dev, dtype=torch.int64)
+    st4, st32 = torch.arange(1, B + 1, device=dev), torch.arange(1, B2 + 1, device=dev)
+    r2t = (torch.arange(T, device=dev, dtype=torch.int32) + 1).view(B, L).contiguous()
+    r2t2 = (torch.arange(B2 * C, device=dev, dtype=torch.int32) + 1).view(B2, C).contiguous()
+    # ---- the seam ----------------------------------------------------------------------------------------------------------
+    for Tn in (8192, 32):
+        y = torch.randn(Tn, W, device=dev, dtype=dt)
+        res = torch.randn(Tn, W, device=dev, dtype=torch.float32)
+        w = torch.zeros(W, device=dev, dtype=dt)
+        t_new = _timed(lambda: ops.outnorm_stream(y, res, w, 1e-5, 1.0))
+        t_old = _timed(lambda: ops.postnorm_stream(y, w, res, 1.0, w, 1e-6))
+        out.append((f"stream += norm(y), copy for the next sublayer, {Tn} rows of {W} (like: stream = norm(alpha stream + scale * y), copy)",
+                    rec(t_new, nbytes=Tn * W * (2 + 4 + 4 + 2.0)), rec(t_old, nbytes=Tn * W * (2 + 4 + 4 + 2.0))))
+    # ---- preparation -------------------------------------------------------------------------------------------------------
+    H, G, D, N, P = s["heads"], s["kv"], s["dim"], s["window"], s["pool"]
+    E = D
+    n_slots = max(T, B2 * C) + 1
+    kp = torch.randn(n_slots, G, D, device=dev, dtype=dt)
+    vp = torch.randn(n_slots, G, E, device=dev, dtype=dt)
+    km = torch.randn(n_slots, G, mean_piece(D, P), device=dev, dtype=dt)
+    vm = torch.randn(n_slots, G, mean_piece(E, P), device=dev, dtype=dt)
+    means = (P, km, vm)
+    nw = torch.ones(D, device=dev, dtype=dt)
+    freq = 10000.0 ** (-2.0 * torch.arange(D // 2, dtype=torch.float32, device=dev) / D)
+    tH, tG, tD, tE = tb["theads"], tb["tkv"], tb["tdim"], tb["tvdim"]
+    tfreq = 10000.0 ** (-2.0 * torch.arange(tD // 2, dtype=torch.float32, device=dev) / tD)
+    tkp, tvp = torch.zeros(n_slots, tG, tD, device=dev, dtype=dt), torch.zeros(n_slots, tG, tE, device=dev, dtype=dt)
+    tqw, tkw, temp = torch.ones(tH * tD, device=dev, dtype=dt), torch.ones(tG * tD, device=dev, dtype=dt), torch.ones(tH, device=dev)
+    for Tn, decode in ((8192, False), (32, True)):
+        p = torch.randn(Tn, (H + G) * D + G * E + H, device=dev, dtype=dt)
+        loc = torch.arange(1, Tn + 1, device=dev) if not decode else r2t2[:, -1].long().contiguous()
+        pos = torch.arange(Tn, device=dev) % L if not decode else torch.full((Tn,), C - 1, device=dev, dtype=torch.int64)
+        tab = ops.angle_table(pos, freq)
+        a = (r2t, rows, lens, q_start, q_len) if not decode else (r2t2, rows2, lens2, None, None)
+        t_new = _timed(lambda: ops.head_norm_rope_kv_store(p, H, G, D, E, H * D, (H + G) * D, nw, nw, 1e-5, tab, D, tab, kp, vp, loc, means,
+                                                           pos, *a))
+        tp = torch.randn(Tn, (tH + tG) * tD + tG * tE, device=dev, dtype=dt)
+        t_old = _timed(lambda: ops.qk_norm_rope_kv_store(tp, tH, tG, tD, tE, tH * tD, (tH + tG) * tD, tqw, tkw, 1e-6, pos, tfreq, tD, False,
+                                                         1.0, temp, tkp, tvp, loc))
+        out.append((f"head norms + rotation of q, k and v + KV store + the means of whole blocks of {P}, {Tn} {'decode rows' if decode else 'tokens'}, "
+                    f"{H} / {G} heads of {D} / {E} (like: norm of q and k over the whole projection + rotation + KV store, {tH} / {tG} heads of "
+                    f"{tD} / {tE})", rec(t_new, nbytes=Tn * 2.0 * (2 * H * D + 2 * G * (D + E)) + (Tn * 2.0 * G * (D + E)) * (1 + 1 / P)),
+                    rec(t_old, nbytes=Tn * 2.0 * (2 * tH * tD + 2 * tG * (tD + tE)))))
+    # ---- attention ---------------------------------------------------------------------------------------------------------
+    q = torch.randn(T, H * D, device=dev, dtype=dt)
+    o = torch.empty(T, H * E, device=dev, dtype=dt)
+    gate = torch.randn(T, H, device=dev, dtype=dt)
+    sink = torch.zeros(H, device=dev)
+    tab = ops.angle_table(torch.arange(T, device=dev) % L, freq)
+    t_new = _timed(lambda: ops.pooled_window_attention_fwd(q, o, kp, vp, means, r2t, rows, lens, q_start, q_len, L, D ** -0.5, N, sink=sink,
+                                                           gate=gate, turn=tab))
+    t_old = _timed(lambda: ops.window_attention_fwd(q, o, kp, vp, r2t, rows, lens, q_start, q_len, L, D ** -0.5, N, 0, None, False, sink))
+    pairs_w = B * sum(min(i + 1, N) for i in range(L))
+    pairs = pairs_w + B * sum(max(0, i - N + 1) // P for i in range(L))
+    out.append((f"prompt attention, {B} x {L} tokens, {H} / {G} heads of {D} / {E}, window {N} + block means of {P}, the result turned back, the "
+                f"heads' gates (like: the window alone, softmax with a sink)",
+                rec(t_new, flops=2.0 * H * (D + E) * pairs), rec(t_old, flops=2.0 * H * (D + E) * pairs_w)))
+    q2 = torch.randn(B2, H * D, device=dev, dtype=dt)
+    o2 = torch.empty(B2, H * E, device=dev, dtype=dt)
+    gate2 = torch.randn(B2, H, device=dev, dtype=dt)
+    tab2 = ops.angle_table(torch.full((B2,), C - 1, device=dev, dtype=torch.int64), freq)
+    nb = max(0, C - N) // P
+    splits = max(1, min(16, 512 // (B2 * G * ((H // G + 15) // 16)), (N + nb) // 128))       # HipAttnBackend.forward_pooled_window's rule on 256 CUs
+    t_new = _timed(lambda: ops.pooled_window_attention_fwd(q2, o2, kp, vp, means, r2t2, rows2, lens2, None, None, 1, D ** -0.5, N, sink=sink,
+                                                           gate=gate2, turn=tab2, n_splits=splits))
+    t_old = _timed(lambda: ops.window_attention_fwd(q2, o2, kp, vp, r2t2, rows2, lens2, None, None, 1, D ** -0.5, N, 0, None, False, sink))
+    out.append((f"decode attention, {B2} requests at {C} tokens, {H} / {G} heads of {D} / {E}, window {N} + block means of {P}, {splits} workgroups "
+                f"share a request's keys (like: the window alone)",
+                rec(t_new, nbytes=B2 * G * (D + E) * 2.0 * (N + nb)), rec(t_old, nbytes=B2 * G * (D + E) * 2.0 * N)))
+    # ---- the recurrences ---------------------------------------------------------------------------------------------------
+    MH, MD, ME = s["mheads"], s["mdim"], s["mvdim"]
+    sizes = [MH * MD, MH * MD, MH * ME, MH * ME, MH, MH]
+    offs = [sum(sizes[:i]) for i in range(6)]
+    width = sum(sizes) + -sum(sizes) % 8
+    ib, fb = torch.zeros(MH, device=dev), torch.zeros(MH, device=dev) + 4.0
+    mnw = torch.ones(MH * ME, device=dev, dtype=dt)
+    S = torch.zeros(B2 + 1, ops.matrix_memory_state_width(MH, MD, ME), device=dev)
+    mp = torch.randn(T, width, device=dev, dtype=dt)
+    t_new = _timed(lambda: ops.matrix_memory(mp, offs, MH, MD, ME, ib, fb, 15.0, mnw, 1e-5, S, st4, lens, q_start, q_len), iters=10, warm=2)
+    SH, SE, SN, SG, taps = tb["sheads"], tb["svdim"], tb["state"], tb["groups"], 4
+    inner, Cc = SH * SE, SH * SE + 2 * SG * SN
+    swidth = 2 * inner + 2 * SG * SN + SH
+    conv_w, conv_b = torch.randn(Cc, taps, device=dev, dtype=dt) * 0.5, torch.zeros(Cc, device=dev, dtype=dt)
+    a_log, dt_bias, dsk = torch.zeros(SH, device=dev) - 1.0, torch.zeros(SH, device=dev), torch.ones(SH, device=dev)
+    onw = torch.ones(inner, device=dev, dtype=dt)
+    sS, cs = torch.zeros(B2 + 1, inner * SN, device=dev), torch.zeros(B2 + 1, (taps - 1) * Cc, device=dev)
+    sp = torch.randn(T, swidth, device=dev, dtype=dt)
+    t_old = _timed(lambda: ops.state_space(sp, 0, inner, inner + Cc, conv_w, conv_b, dt_bias, a_log, dsk, onw, 1, 1e-5, sS, cs, st4, lens,
+                                           q_start, q_len, SH, SG, SN, SE), iters=5, warm=1)
+    out.append((f"matrix memory over {B} x {L} tokens, {MH} heads of {MD} x {ME} (gates, chunks of 64 tokens on the matrix cores, division, norm, gate; "
+                f"priced like the recurrence it is: 4 flop per element of S and token on the vector units; like: state-space recurrence, {SH} "
+                f"heads of {SN} x {SE}, 4 flop per element)",
+                rec(t_new, nbytes=T * 2.0 * (width + MH * ME), vflops=4.0 * T * MH * MD * ME),
+                rec(t_old, nbytes=T * 2.0 * (swidth + inner), vflops=4.0 * T * inner * SN)))
+    mpd = torch.randn(B2, width, device=dev, dtype=dt)
+    t_new = _timed(lambda: ops.matrix_memory(mpd, offs, MH, MD, ME, ib, fb, 15.0, mnw, 1e-5, S, st32, lens2, None, None))
+    spd = torch.randn(B2, swidth, device=dev, dtype=dt)
+    t_old = _timed(lambda: ops.state_space(spd, 0, inner, inner + Cc, conv_w, conv_b, dt_bias, a_log, dsk, onw, 1, 1e-5, sS, cs, st32, lens2,
+                                           None, None, SH, SG, SN, SE))
+    out.append((f"matrix-memory decode step, {B2} requests (reads and writes {MH * MD * ME * 4 / 1e6:.1f} MB of state per request; like: "
+                f"state-space decode step, {inner * SN * 4 / 1e6:.1f} MB per request)",
+                rec(t_new, nbytes=B2 * MH * MD * ME * 4.0 * 2), rec(t_old, nbytes=B2 * inner * SN * 4.0 * 2)))
+    return out
+
+
+def main_gukidra(args) -> dict:
+    from semi_pd_amd.models.gukidra import gukidra_uniform
+    from semi_pd_amd.models.tibenex import tibenex_uniform
+    dev = torch.device("cuda:0")
+    torch.cuda.set_device(dev)
+    names = [n for n in (getattr(args, "arch_sizes", "") or ",".join(GUKIDRA_SIZES)).split(",") if n]
+    result = {"what": "Gukidra next to Tibenex at equal layer sizes", "dtype": "bf16", "data": "synthetic", "models": {}, "kernels": {}}
+    for name in names:
+        s, tb = GUKIDRA_SIZES[name], TIBENEX_SIZES[name]
+        result["kernels"][name] = [
+            {"kernel": what, "gukidra": new, "like": old,
+             "roofline_fraction_ratio": round(new["of_roofline"] / max(old["of_roofline"], 1e-9), 2)}
+            for what, new, old in _gukidra_kernel_pairs(s, tb, dev)]
+        gcfg = gukidra_uniform(s["vocab"], s["hidden"], "amsm", s["ff"], s["heads"], s["kv"], s["dim"], s["dim"], s["window"], s["pool"],
+                               s["mheads"], s["mdim"], s["mvdim"])
+        tcfg = tibenex_uniform(tb["vocab"], tb["hidden"], "lmam", tb["ff"], tb["theads"], tb["tkv"], tb["tdim"], tb["tvdim"], tb["rot"],
+                               tb["rank"], tb["qrank"], tb["sheads"], tb["svdim"], tb["state"], tb["groups"], latent_heads=tb["heads"],
+                               latent_dim=tb["dim"], latent_vdim=tb["vdim"])
+        result["models"][name] = {
+            "layers": 4,
+            "gukidra": _model_throughput(gcfg, 2048, 4, 32, 1100, 20),
+            "tibenex": _model_throughput(tcfg, 2048, 4, 32, 1100, 20)}
+    print(json.dumps(result), flush=True)
+    return result
+
+
 def main(args) -> dict:
+    if getattr(args, "arch_design", "kudirax") == "gukidra":
+        return main_gukidra(args)
     if getattr(args, "arch_design", "kudirax") == "tibenex":
         return main_tibenex(args)
     if getattr(args, "arch_design", "kudirax") == "tigotar":
