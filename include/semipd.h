@@ -1012,15 +1012,17 @@ int semipd_angle_table(const int64_t* positions, const float* freq, int half, in
 int semipd_head_norm_rope_kv_store(void* qkv, int64_t ld, int64_t num_tokens, int num_q_heads, int num_kv_heads, int qk_dim,
                                    int v_dim, int64_t k_off, int64_t v_off, const void* q_weight, const void* k_weight, float eps,
                                    const float* qk_angles, int rot_dims, const float* v_angles, void* k_pool, void* v_pool,
-                                   const int64_t* loc, const int64_t* positions, int pool, void* k_means, void* v_means, int k_piece,
-                                   int v_piece, const int32_t* req_to_token, int64_t req_to_token_stride,
+                                   const int64_t* loc, const int64_t* positions, int pool, void* k_means, void* v_means,
+                                   int64_t mean_slots, int k_piece, int v_piece, const int32_t* req_to_token, int64_t req_to_token_stride,
                                    const int64_t* req_pool_indices, const int64_t* seq_lens, const int32_t* q_start,
                                    const int32_t* q_len, int64_t batch, int dtype, void* stream);
 /* The means of the blocks of `pool` tokens that the batch's rows complete, over the rows the pools hold, fp32 sums in token
  * order, one rounding.  A mean is cut into pieces of k_piece / v_piece elements (powers of two, >= 8, piece * pool >= the head
- * size); piece i of block b lies at the slot of token b * pool + i: k_means [slots, num_kv_heads, k_piece], v_means likewise. */
+ * size); piece i of block b lies at the slot of token b * pool + i: k_means [num_kv_heads, mean_slots, k_piece], v_means
+ * likewise. */
 int semipd_block_means(const void* k_pool, const void* v_pool, int num_kv_heads, int qk_dim, int v_dim, int pool, void* k_means,
-                       void* v_means, int k_piece, int v_piece, const int32_t* req_to_token, int64_t req_to_token_stride,
+                       void* v_means, int64_t mean_slots, int k_piece, int v_piece, const int32_t* req_to_token,
+                       int64_t req_to_token_stride,
                        const int64_t* req_pool_indices, const int64_t* seq_lens, const int32_t* q_start, const int32_t* q_len,
                        int64_t batch, int64_t num_tokens, int dtype, void* stream);
 /* Sliding-window softmax attention (last `window` positions, 0: all) that sees, in the same softmax, the means of the blocks of
@@ -1029,14 +1031,14 @@ int semipd_block_means(const void* k_pool, const void* v_pool, int num_kv_heads,
  * sigmoid(gate[row, head]) (NULL: not).  n_splits / partial as in semipd_latent_attention (partial fp32
  * [rows, heads, n_splits, v_dim + 2]). */
 int semipd_pooled_window_attention(const void* q, int64_t q_ld, const void* gate, int64_t gate_ld, void* out, int64_t out_ld,
-                                   const void* k_pool, const void* v_pool, const void* k_means, const void* v_means, int k_piece,
-                                   int v_piece, const int32_t* req_to_token, int64_t req_to_token_stride,
+                                   const void* k_pool, const void* v_pool, const void* k_means, const void* v_means,
+                                   int64_t mean_slots, int k_piece, int v_piece, const int32_t* req_to_token, int64_t req_to_token_stride,
                                    const int64_t* req_pool_indices, const int64_t* seq_lens, const int32_t* q_start,
                                    const int32_t* q_len, int64_t batch, int64_t num_tokens, int64_t max_q_len, int num_q_heads,
                                    int num_kv_heads, int qk_dim, int v_dim, float scale, int window, int pool, const float* sink,
                                    const float* turn, int n_splits, float* partial, int form, int dtype, void* stream);
-/* fp32 elements of a work row and of a request's state of semipd_matrix_memory. */
-int64_t semipd_matrix_memory_work_width(int num_heads, int v_dim);
+/* fp32 elements of the workspace and of a request's state of semipd_matrix_memory. */
+int64_t semipd_matrix_memory_workspace(int64_t num_tokens, int num_heads, int v_dim);
 int64_t semipd_matrix_memory_state_width(int num_heads, int qk_dim, int v_dim);
 /* Matrix memory with exponential gates behind its projection GEMM: rows [q | k | v | g | i | f] at the given columns, gate
  * biases fp32 [H], norm_w [H * v_dim]; state fp32 [slots, state width] (S [H, qk_dim, v_dim] | n [H, qk_dim] | m [H]) is a column
@@ -1044,7 +1046,7 @@ int64_t semipd_matrix_memory_state_width(int num_heads, int qk_dim, int v_dim);
  * description as in semipd_local_attention.  form: 0 by shape and type, 1 token by token, 2 the matrix-core form. */
 int semipd_matrix_memory(const void* proj, int64_t ld, int64_t q_off, int64_t k_off, int64_t v_off, int64_t g_off, int64_t i_off,
                          int64_t f_off, const float* i_bias, const float* f_bias, float gate_cap, const void* norm_w, float eps,
-                         float* work, int64_t work_ld, float* state, int64_t state_ld, const int64_t* state_indices,
+                         float* work, int64_t work_elems, float* state, int64_t state_ld, const int64_t* state_indices,
                          const int64_t* seq_lens, const int32_t* q_start, const int32_t* q_len, int64_t batch, int64_t num_tokens,
                          int num_heads, int qk_dim, int v_dim, float q_scale, void* out, int64_t out_ld, int form, int dtype,
                          void* stream);

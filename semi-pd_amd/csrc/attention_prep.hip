@@ -9,7 +9,7 @@
 //  * block_means_kernel: the mean key and the mean value of every block of `pool` tokens that the batch completes, as the
 //    pools hold them.  A mean is not kept as a row of its own: it is cut into pieces of 2^sh elements and piece i lies in the
 //    mean pools at the slot of the block's token i -- about 1 / pool of the token rows' memory, handed out and given back with
-//    the tokens' own slots.  Batches of one row per request take their means inside the preparation launch where that has
+//    the tokens' own slots, and one contiguous row per head where the tokens' slots are neighbours.  Batches of one row per request take their means inside the preparation launch where that has
 //    the vector form.
 #include "common.h"
 
@@ -40,7 +40,8 @@ struct HeadPrepArgs {
   const int64_t* req_pool_indices; const int64_t* seq_lens;
   const int32_t* q_start; const int32_t* q_len; int64_t batch;
   int pool, k_sh, v_sh;                      // pool 0: no means
-  void* kb_pool; void* vb_pool;              // rows of G << k_sh, G << v_sh elements
+  void* kb_pool; void* vb_pool;              // [G, mean_slots, 1 << sh]
+  int64_t mean_slots;
 };
 
 // One wave per (row, head of q | k | v).
@@ -187,9 +188,9 @@ __global__ void __launch_bounds__(256) head_norm_rope_kv_store_vec_kernel(HeadPr
       oy.e[i] = Elem<T>::from_f(my[i] * inv);
     }
     const int sh = is_v ? a.v_sh : a.k_sh, mask = (1 << sh) - 1;
-    T* means = (T*)(is_v ? a.vb_pool : a.kb_pool) + ((int64_t)head << sh);
-    store16(means + ((int64_t)slots[e0 >> sh] * G << sh) + (e0 & mask), ox);
-    store16(means + ((int64_t)slots[e1 >> sh] * G << sh) + (e1 & mask), oy);
+    T* means = (T*)(is_v ? a.vb_pool : a.kb_pool) + ((head * a.mean_slots) << sh);
+    store16(means + ((int64_t)slots[e0 >> sh] << sh) + (e0 & mask), ox);
+    store16(means + ((int64_t)slots[e1 >> sh] << sh) + (e1 & mask), oy);
   }
 }
 
@@ -250,7 +251,7 @@ __global__ void __launch_bounds__(256) block_means_kernel(HeadPrepArgs a) {
       for (; j < P; ++j) m[0] += Elem<T>::to_f(src[(int64_t)slots[j] * ld]);
     }
     const int sh = is_v ? a.v_sh : a.k_sh;
-    T* dst = (T*)(is_v ? a.vb_pool : a.kb_pool) + (((int64_t)slots[e >> sh] * G + head) << sh) + (e & ((1 << sh) - 1));
+    T* dst = (T*)(is_v ? a.vb_pool : a.kb_pool) + ((head * a.mean_slots + slots[e >> sh]) << sh) + (e & ((1 << sh) - 1));
     if constexpr (V > 1) {
       Vec16<T> o;
 #pragma unroll
@@ -302,7 +303,7 @@ static int check_means(const char* what, const HeadPrepArgs& a, int k_piece, int
                        v_piece >= 8,
                    SEMIPD_ESHAPE, "%s: pieces of %d / %d elements (powers of two from 8 up that cover %d / %d in %d tokens)", what, k_piece,
                    v_piece, a.D, a.E, a.pool);
-  SEMIPD_CHECK_ARG(a.kb_pool && a.vb_pool && a.k_pool && a.v_pool && a.req_to_token && a.req_pool_indices && a.seq_lens, SEMIPD_EINVAL,
+  SEMIPD_CHECK_ARG(a.kb_pool && a.vb_pool && a.mean_slots > 0 && a.k_pool && a.v_pool && a.req_to_token && a.req_pool_indices && a.seq_lens, SEMIPD_EINVAL,
                    "%s: null pointer", what);
   SEMIPD_CHECK_ARG((a.q_start == nullptr) == (a.q_len == nullptr) && (a.q_start != nullptr || a.num_tokens == a.batch), SEMIPD_EINVAL,
                    "%s: q_start and q_len come together; without them one row per request", what);
@@ -313,7 +314,7 @@ extern "C" int semipd_head_norm_rope_kv_store(void* qkv, int64_t ld, int64_t num
                                               int v_dim, int64_t k_off, int64_t v_off, const void* q_weight, const void* k_weight,
                                               float eps, const float* qk_angles, int rot_dims, const float* v_angles, void* k_pool,
                                               void* v_pool, const int64_t* loc, const int64_t* positions, int pool, void* k_means,
-                                              void* v_means, int k_piece, int v_piece, const int32_t* req_to_token,
+                                              void* v_means, int64_t mean_slots, int k_piece, int v_piece, const int32_t* req_to_token,
                                               int64_t req_to_token_stride, const int64_t* req_pool_indices, const int64_t* seq_lens,
                                               const int32_t* q_start, const int32_t* q_len, int64_t batch, int dtype, void* stream) {
   SEMIPD_CHECK_ARG(num_tokens >= 0 && num_q_heads >= 0 && num_kv_heads >= 0 && num_q_heads + num_kv_heads > 0 && qk_dim > 0,
@@ -331,7 +332,7 @@ extern "C" int semipd_head_norm_rope_kv_store(void* qkv, int64_t ld, int64_t num
   SEMIPD_CHECK_ARG(pool == 0 || num_kv_heads > 0, SEMIPD_EINVAL, "head_norm_rope_kv_store: block means without keys");
   HeadPrepArgs a{qkv, ld, num_tokens, num_q_heads, num_kv_heads, qk_dim, v_dim, k_off, v_off, q_weight, k_weight, eps, qk_angles,
                  rot_dims, v_angles, k_pool, v_pool, loc, positions, req_to_token, req_to_token_stride, req_pool_indices, seq_lens,
-                 q_start, q_len, batch, pool, piece_shift(k_piece), piece_shift(v_piece), k_means, v_means};
+                 q_start, q_len, batch, pool, piece_shift(k_piece), piece_shift(v_piece), k_means, v_means, mean_slots};
   if (pool > 0) {
     const int rc = check_means("head_norm_rope_kv_store", a, k_piece, v_piece);
     if (rc) return rc;
@@ -379,7 +380,7 @@ extern "C" int semipd_head_norm_rope_kv_store(void* qkv, int64_t ld, int64_t num
 }
 
 extern "C" int semipd_block_means(const void* k_pool, const void* v_pool, int num_kv_heads, int qk_dim, int v_dim, int pool,
-                                  void* k_means, void* v_means, int k_piece, int v_piece, const int32_t* req_to_token,
+                                  void* k_means, void* v_means, int64_t mean_slots, int k_piece, int v_piece, const int32_t* req_to_token,
                                   int64_t req_to_token_stride, const int64_t* req_pool_indices, const int64_t* seq_lens,
                                   const int32_t* q_start, const int32_t* q_len, int64_t batch, int64_t num_tokens, int dtype,
                                   void* stream) {
@@ -388,7 +389,8 @@ extern "C" int semipd_block_means(const void* k_pool, const void* v_pool, int nu
   if (batch == 0 || num_tokens == 0) return 0;
   HeadPrepArgs a{nullptr, 0, num_tokens, 0, num_kv_heads, qk_dim, v_dim, 0, 0, nullptr, nullptr, 0.f, nullptr, 0, nullptr,
                  const_cast<void*>(k_pool), const_cast<void*>(v_pool), nullptr, nullptr, req_to_token, req_to_token_stride,
-                 req_pool_indices, seq_lens, q_start, q_len, batch, pool, piece_shift(k_piece), piece_shift(v_piece), k_means, v_means};
+                 req_pool_indices, seq_lens, q_start, q_len, batch, pool, piece_shift(k_piece), piece_shift(v_piece), k_means, v_means,
+                 mean_slots};
   int rc = check_means("block_means", a, k_piece, v_piece);
   if (rc) return rc;
   rc = launch_block_means(a, dtype, as_stream(stream));

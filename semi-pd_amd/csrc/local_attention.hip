@@ -484,10 +484,10 @@ struct LocalAttnArgs {
   int v_shared;                    // 1: the value row of a slot is ONE head of E elements that every key/value head's queries read
   // block means (POOL kernels): blocks of `pool` tokens that lie wholly in front of the window are seen through one key and
   // one value each.  The mean of block b is cut into pieces of 2^k_sh (2^v_sh) elements; piece i lies in the mean pools at the
-  // slot of token b * pool + i (rows of kb_ld / vb_ld elements, kv head g's piece at g << k_sh)
+  // slot of token b * pool + i: [G, mean_slots, piece] (neighbouring slots: a whole mean is one contiguous row)
   int pool;                        // 0: no blocks
   const void* kb_pool; const void* vb_pool;
-  int64_t kb_ld, vb_ld;
+  int64_t mean_slots;
   int k_sh, v_sh;
   const float* turn;               // POOL kernels: [rows, E / 2] (cos, sin): the result is turned BACK by these angles, pairs (m, m + E / 2)
 };
@@ -560,8 +560,8 @@ __global__ void __launch_bounds__(256) local_attention_rows_kernel(LocalAttnArgs
   constexpr int V = Elem<T>::kVec;
   // the kept first positions (none without a window) or the block means, then the range that ends at the query
   const int64_t n_blocks = POOL ? blocks_seen(a, pos) : 0;
-  const T* kb = POOL ? (const T*)a.kb_pool + ((int64_t)g << a.k_sh) : nullptr;
-  const T* vb = POOL ? (const T*)a.vb_pool + ((int64_t)g << a.v_sh) : nullptr;
+  const T* kb = POOL ? (const T*)a.kb_pool + ((g * a.mean_slots) << a.k_sh) : nullptr;
+  const T* vb = POOL ? (const T*)a.vb_pool + ((g * a.mean_slots) << a.v_sh) : nullptr;
   for (int seg = (n_first > 0 || n_blocks > 0) ? 0 : 1; seg < 2; ++seg) {
     const bool blk = POOL && seg == 0;
     const int64_t j_begin = seg == 0 ? 0 : lo, j_last = seg == 0 ? (POOL ? n_blocks : n_first) - 1 : pos;
@@ -577,13 +577,13 @@ __global__ void __launch_bounds__(256) local_attention_rows_kernel(LocalAttnArgs
           float dot = 0.f;
           if ((D % V) == 0) {
             for (int d = 0; d < D; d += V) {
-              const Vec16<T> kv = load16(kb + (int64_t)brow[d >> a.k_sh] * a.kb_ld + (d & kmask));
+              const Vec16<T> kv = load16(kb + ((int64_t)brow[d >> a.k_sh] << a.k_sh) + (d & kmask));
 #pragma unroll
               for (int u = 0; u < V; ++u) dot += q_lds[wave][d + u] * Elem<T>::to_f(kv.e[u]);
             }
           } else {
             for (int d = 0; d < D; ++d)
-              dot += q_lds[wave][d] * Elem<T>::to_f(kb[(int64_t)brow[d >> a.k_sh] * a.kb_ld + (d & kmask)]);
+              dot += q_lds[wave][d] * Elem<T>::to_f(kb[((int64_t)brow[d >> a.k_sh] << a.k_sh) + (d & kmask)]);
           }
           s = capped(dot, a.scale, a.cap);
         }
@@ -623,7 +623,7 @@ __global__ void __launch_bounds__(256) local_attention_rows_kernel(LocalAttnArgs
 #pragma unroll
           for (int u = 0; u < NA; ++u) {
             const int e = lane + 64 * u;
-            if (e < E) acc[u] += pj * Elem<T>::to_f(vb[(int64_t)brow[e >> a.v_sh] * a.vb_ld + (e & vmask)]);
+            if (e < E) acc[u] += pj * Elem<T>::to_f(vb[((int64_t)brow[e >> a.v_sh] << a.v_sh) + (e & vmask)]);
           }
           continue;
         }
@@ -711,48 +711,75 @@ template <int ND> struct KFrags {
   Frag16 a[ND], b[ND];
 };
 
-// Where the rows of key j lie.  TokenRows: key j is position j of the sequence, its slot from the copy of this part of the
-// request's row in LDS when the caller made one (the load of a row of the pool then waits for nothing but itself), else from
-// the table.
+// Where the rows of key j lie.  A walk asks for the keys of one step of 32 at a time (`step`).
+// TokenRows: key j is position j of the sequence, its slot from the copy of this part of the request's row in LDS when the
+// caller made one (the load of a row of the pool then waits for nothing but itself), else from the table.
 template <typename T> struct TokenRows {
   const T* kp; int64_t kstride;
   const T* vp; int64_t vstride;
   const int32_t* row; const int32_t* idx_lds; int64_t idx_base;
-  __device__ __forceinline__ int64_t slot(int64_t j) const { return idx_lds ? idx_lds[j - idx_base] : row[j]; }
-  __device__ __forceinline__ bool have(int64_t j, int64_t j_end) const { return j <= j_end; }
-  __device__ __forceinline__ const T* k(int64_t j, int e) const { return kp + slot(j) * kstride + e; }
-  __device__ __forceinline__ const T* v(int64_t j, int e) const { return vp + slot(j) * vstride + e; }
-  // a lane's K row: looked up once for all of its pieces (keys that are not there: the dummy slot)
   struct KRow {
     const T* p;
     __device__ __forceinline__ const T* at(int e) const { return p + e; }
   };
-  __device__ __forceinline__ KRow krow(int64_t j, int64_t j_end) const { return KRow{kp + (j <= j_end ? slot(j) : 0) * kstride}; }
+  struct Step {
+    const TokenRows& r; int64_t j_end;
+    __device__ __forceinline__ bool have(int64_t j) const { return j <= j_end; }
+    __device__ __forceinline__ const T* k(int64_t j, int e) const { return r.kp + r.slot(j) * r.kstride + e; }
+    __device__ __forceinline__ const T* v(int64_t j, int e) const { return r.vp + r.slot(j) * r.vstride + e; }
+    // a lane's K row: looked up once for all of its pieces (a key that is not there: the dummy slot)
+    __device__ __forceinline__ KRow krow(int64_t j) const { return KRow{r.kp + (j <= j_end ? r.slot(j) : 0) * r.kstride}; }
+  };
+  __device__ __forceinline__ int64_t slot(int64_t j) const { return idx_lds ? idx_lds[j - idx_base] : row[j]; }
+  __device__ __forceinline__ Step step(int64_t, int64_t j_end) const { return Step{*this, j_end}; }
 };
 // PooledRows: keys 0 .. nb - 1 are the block means (nb_pad: nb up to whole steps of 32 keys, so that a step is all blocks or
-// all tokens), key nb_pad + i is position tok0 + i.
+// all tokens), key nb_pad + i is position tok0 + i.  Element e of key j lies at the slot of position j * mul + add + (e >> shift),
+// element e & mask of that slot's row: pieces of a mean beside the block's tokens, or (mul 1, shift 31, mask ~0) a token's row;
+// which of the two is the same for a whole step and every lane.
 template <typename T> struct PooledRows {
   TokenRows<T> tok;
-  const T* kb; int64_t kb_ld;
-  const T* vb; int64_t vb_ld;
+  bool blk_lds;                    // whether the copy of the row in LDS serves the blocks' lookups too (it may hold the window only)
+  const T* kb; const T* vb;
   int k_sh, v_sh, pool;
   int64_t nb, nb_pad, tok0;
-  __device__ __forceinline__ bool have(int64_t j, int64_t j_end) const { return j < nb_pad ? j < nb : j <= j_end; }
-  __device__ __forceinline__ const T* k(int64_t j, int e) const {
-    if (j < nb_pad) return kb + tok.slot(j * pool + (e >> k_sh)) * kb_ld + (e & ((1 << k_sh) - 1));
-    return tok.k(tok0 + j - nb_pad, e);
-  }
-  __device__ __forceinline__ const T* v(int64_t j, int e) const {
-    if (j < nb_pad) return vb + tok.slot(j * pool + (e >> v_sh)) * vb_ld + (e & ((1 << v_sh) - 1));
-    return tok.v(tok0 + j - nb_pad, e);
-  }
-  struct KRow {
-    const PooledRows* r; int64_t j; const T* p;      // p: the row of a token, null for a block
-    __device__ __forceinline__ const T* at(int e) const { return p ? p + e : r->k(j, e); }
+  struct Step {
+    const T* kp; const T* vp;
+    int64_t kld, vld;
+    const int32_t* row; const int32_t* idx_lds;
+    int idx_base;                  // position of idx_lds[0]
+    bool lds;
+    int mul, add, k_sh, v_sh, k_mask, v_mask, last;      // last: the last key of the step's kind
+    bool blk;
+    __device__ __forceinline__ int64_t slot(int pos) const { return lds ? idx_lds[pos - idx_base] : row[pos]; }
+    struct KRow {
+      const Step& s; int pos; bool there; const T* p;
+      __device__ __forceinline__ const T* at(int e) const {
+        if (!s.blk) return p + e;
+        return s.kp + (there ? s.slot(pos + (e >> s.k_sh)) : 0) * s.kld + (e & s.k_mask);
+      }
+    };
+    __device__ __forceinline__ bool have(int64_t j) const { return (int)j <= last; }
+    __device__ __forceinline__ const T* k(int64_t j, int e) const {
+      return kp + slot((int)j * mul + add + (e >> k_sh)) * kld + (e & k_mask);
+    }
+    __device__ __forceinline__ const T* v(int64_t j, int e) const {
+      return vp + slot((int)j * mul + add + (e >> v_sh)) * vld + (e & v_mask);
+    }
+    __device__ __forceinline__ KRow krow(int64_t j) const {
+      const bool there = (int)j <= last;
+      const int pos = (int)j * mul + add;
+      return KRow{*this, pos, there, blk ? nullptr : kp + (there ? slot(pos) : 0) * kld};
+    }
   };
-  __device__ __forceinline__ KRow krow(int64_t j, int64_t j_end) const {
-    if (!have(j, j_end)) return KRow{this, j, tok.kp};                      // the dummy slot
-    return j < nb_pad ? KRow{this, j, nullptr} : KRow{this, j, tok.k(tok0 + j - nb_pad, 0)};
+  __device__ __forceinline__ Step step(int64_t j0, int64_t j_end) const {
+    const bool blk = __builtin_amdgcn_readfirstlane((int)(j0 < nb_pad)) != 0;
+    const int base = (int)tok.idx_base;
+    if (blk)
+      return Step{kb, vb, (int64_t)1 << k_sh, (int64_t)1 << v_sh, tok.row, tok.idx_lds, base, blk_lds, pool, 0, k_sh, v_sh,
+                  (1 << k_sh) - 1, (1 << v_sh) - 1, (int)nb - 1, true};
+    return Step{tok.kp, tok.vp, tok.kstride, tok.vstride, tok.row, tok.idx_lds, base, tok.idx_lds != nullptr, 1, (int)(tok0 - nb_pad),
+                31, 31, -1, -1, (int)j_end, false};
   }
 };
 
@@ -804,11 +831,12 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
     }
   };
   auto load_v = [&](int64_t j0) {
+    const auto at = rows.step(j0, j_end);
 #pragma unroll
     for (int i = 0; i < NV; ++i)
       if (v_key[i] >= 0) {
         const int64_t j = j0 + v_key[i];
-        vr[i] = rows.have(j, j_end) ? *reinterpret_cast<const uint4*>(rows.v(j, v_ec[i] * 8)) : uint4{0u, 0u, 0u, 0u};
+        vr[i] = at.have(j) ? *reinterpret_cast<const uint4*>(at.v(j, v_ec[i] * 8)) : uint4{0u, 0u, 0u, 0u};
       }
   };
   auto store_v = [&](int buf) {        // buf: which pair of tiles (a lone wave has one)
@@ -822,16 +850,18 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
     }
   };
   auto load_k_rows = [&](int64_t j0) {
+    const auto at = rows.step(j0, j_end);
 #pragma unroll
     for (int i = 0; i < NK; ++i)
       if (k_key[i] >= 0) {
         const int64_t j = j0 + k_key[i];
-        kr[i] = rows.have(j, j_end) ? *reinterpret_cast<const uint4*>(rows.k(j, k_ec[i] * 8)) : uint4{0u, 0u, 0u, 0u};
+        kr[i] = at.have(j) ? *reinterpret_cast<const uint4*>(at.k(j, k_ec[i] * 8)) : uint4{0u, 0u, 0u, 0u};
       }
   };
   auto load_k = [&](int64_t j0, auto& k) {
     const int64_t ja = j0 + r, jb = ja + 16;
-    const auto pa = rows.krow(ja, j_end), pb = rows.krow(jb, j_end);
+    const auto at = rows.step(j0, j_end);
+    const auto pa = at.krow(ja), pb = at.krow(jb);
 #pragma unroll
     for (int kk = 0; kk < ND; ++kk)
       if (kk < nd) {
@@ -951,7 +981,7 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
 
 // Prompt portions: 64 query rows of one request and one head per workgroup, 16 per wave.
 template <typename T, int ND, int NE, bool SIG, bool POOL>
-__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 4 ? (POOL ? 3 : 4) : 1))) local_attention_mfma_kernel(LocalAttnArgs a) {
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 4 ? 4 : 1))) local_attention_mfma_kernel(LocalAttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) uint8_t v_lds[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
   // Workgroup -> (kv head, 64-row tile, q head of the group), the last fastest.  Consecutive workgroup ids go round the
@@ -1023,8 +1053,8 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 
     // one walk: the blocks that the tile's last row sees, then the positions of the tile's window range
     const int64_t nb = blocks_seen(a, blk_hi), nb_pad = (nb + 31) / 32 * 32;
     const int64_t my_nb = blocks_seen(a, my_pos), w_nb = blocks_seen(a, w_hi);
-    const PooledRows<T> prows{rows, (const T*)a.kb_pool + ((int64_t)gk << a.k_sh), a.kb_ld,
-                              (const T*)a.vb_pool + ((int64_t)gk << a.v_sh), a.vb_ld, a.k_sh, a.v_sh, a.pool, nb, nb_pad, blk_lo};
+    const PooledRows<T> prows{rows, false, (const T*)a.kb_pool + ((gk * a.mean_slots) << a.k_sh),
+                              (const T*)a.vb_pool + ((gk * a.mean_slots) << a.v_sh), a.k_sh, a.v_sh, a.pool, nb, nb_pad, blk_lo};
     key_walk<T, ND, NE, 256, true, false>(
         st, qf, nd, ne, E, prows, 0, nb_pad + blk_hi - blk_lo, 32, v_lds, tid, a.scale, a.cap,
         [&](int64_t j) {
@@ -1205,7 +1235,12 @@ __global__ void __launch_bounds__(64 * NW) local_attention_decode_kernel(LocalAt
     p_lo = lo < nb_pad ? lo * a.pool : lo_q + lo - nb_pad;
     p_hi = pos < nb_pad ? (pos < nb ? pos + 1 : nb) * a.pool - 1 : lo_q + pos - nb_pad;
   }
-  const bool idx_fits = p_hi - p_lo < kIdxLds;
+  bool idx_fits = p_hi - p_lo < kIdxLds;
+  const bool blk_idx = idx_fits;
+  if (POOL && !idx_fits && pos >= nb_pad) {          // not all of it: the window's part
+    p_lo = lo > nb_pad ? lo_q + lo - nb_pad : lo_q;
+    idx_fits = p_hi - p_lo < kIdxLds;
+  }
   if (idx_fits) {
     for (int64_t j = p_lo + tid; j <= p_hi; j += 64 * NW) idx_lds[j - p_lo] = row[j];
     __syncthreads();
@@ -1214,8 +1249,8 @@ __global__ void __launch_bounds__(64 * NW) local_attention_decode_kernel(LocalAt
   const TokenRows<T> rows{(const T*)a.k_pool + (int64_t)gk * D, a.k_ld, (const T*)a.v_pool + (a.v_shared ? 0 : (int64_t)gk * E),
                           a.v_ld, row, idx_fits ? idx_lds : nullptr, p_lo};
   if constexpr (POOL) {
-    const PooledRows<T> prows{rows, (const T*)a.kb_pool + ((int64_t)gk << a.k_sh), a.kb_ld,
-                              (const T*)a.vb_pool + ((int64_t)gk << a.v_sh), a.vb_ld, a.k_sh, a.v_sh, a.pool, nb, nb_pad, lo_q};
+    const PooledRows<T> prows{rows, blk_idx, (const T*)a.kb_pool + ((gk * a.mean_slots) << a.k_sh),
+                              (const T*)a.vb_pool + ((gk * a.mean_slots) << a.v_sh), a.k_sh, a.v_sh, a.pool, nb, nb_pad, lo_q};
     key_walk<T, ND, NE, 64, false, false>(st, qf, nd, ne, E, prows, lo + 32 * wave, pos, 32 * NW, mine_b, lane, a.scale, a.cap,
                                           [&](int64_t j) { return j < nb_pad ? j < nb && j <= pos : j <= pos; },
                                           [&](int64_t) { return true; }, r, g);
@@ -1545,7 +1580,8 @@ static int launch_local_attention(LocalAttnArgs a, int64_t max_q_len, int form, 
 // sink term, the result turned back by the query's own angles and one gate per head.
 extern "C" int semipd_pooled_window_attention(const void* q, int64_t q_ld, const void* gate, int64_t gate_ld, void* out,
                                               int64_t out_ld, const void* k_pool, const void* v_pool, const void* k_means,
-                                              const void* v_means, int k_piece, int v_piece, const int32_t* req_to_token,
+                                              const void* v_means, int64_t mean_slots, int k_piece, int v_piece,
+                                              const int32_t* req_to_token,
                                               int64_t req_to_token_stride, const int64_t* req_pool_indices,
                                               const int64_t* seq_lens, const int32_t* q_start, const int32_t* q_len,
                                               int64_t batch, int64_t num_tokens, int64_t max_q_len, int num_q_heads,
@@ -1559,7 +1595,7 @@ extern "C" int semipd_pooled_window_attention(const void* q, int64_t q_ld, const
                    "pooled_window_attention: up to 64 slices of the keys, with room for their partial sums");
   int k_sh = 0, v_sh = 0;
   if (pool > 0) {
-    SEMIPD_CHECK_ARG(k_means && v_means, SEMIPD_EINVAL, "pooled_window_attention: blocks without their means");
+    SEMIPD_CHECK_ARG(k_means && v_means && mean_slots > 0, SEMIPD_EINVAL, "pooled_window_attention: blocks without their means");
     while ((1 << k_sh) < k_piece) ++k_sh;
     while ((1 << v_sh) < v_piece) ++v_sh;
     const int unit = dtype == SEMIPD_F32 ? 4 : 8;
@@ -1571,7 +1607,7 @@ extern "C" int semipd_pooled_window_attention(const void* q, int64_t q_ld, const
   LocalAttnArgs a{q, q_ld, gate, gate_ld, out, out_ld, k_pool, v_pool, req_to_token, req_to_token_stride, req_pool_indices,
                   seq_lens, q_start, q_len, batch, num_tokens, num_q_heads, num_kv_heads, qk_dim, v_dim, sink, scale, 0.f,
                   0, 0, window, 0, nullptr, 0, 1.0f, 0, 0, n_splits, partial, 0, pool, k_means, v_means,
-                  (int64_t)num_kv_heads << k_sh, (int64_t)num_kv_heads << v_sh, k_sh, v_sh, turn};
+                  mean_slots, k_sh, v_sh, turn};
   return launch_attention<true>(a, max_q_len, form, dtype, stream);
 }
 

@@ -378,13 +378,13 @@ class HipAttnBackend(AttentionBackend):
         if forward_batch.forward_mode.is_decode():
             q_start = q_len = None
             max_q = 1
-            # (requests x key/value heads x groups of 16 heads) workgroups: below two per CU the keys of a request -- its
+            # (requests x key/value heads x groups of 16 heads) workgroups: below one per CU the keys of a request -- its
             # window and the blocks in front of it -- are shared out over several, about 128 keys each at least
             wgs = T * layer.tp_k_head_num * ((layer.tp_q_head_num // layer.tp_k_head_num + 15) // 16)
             keys = self._decode_len_bound
             if layer.window:
                 keys = min(keys, layer.window) + (max(0, keys - layer.window) // layer.pool if layer.pool else 0)
-            n_splits = max(1, min(16, (2 * max(1, self.num_cus)) // max(wgs, 1), keys // 128))
+            n_splits = max(1, min(16, max(1, self.num_cus) // max(wgs, 1), keys // 128))
             n_splits = int(os.environ.get("SEMIPD_POOLED_DECODE_SPLITS", n_splits))
         else:
             q_start, q_len = forward_batch.extend_start_loc, forward_batch.extend_seq_lens

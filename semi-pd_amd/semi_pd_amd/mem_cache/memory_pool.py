@@ -178,7 +178,7 @@ class MHATokenToKVPool:
     part, and the latent is the value); such a pool has no value regions, its value buffers are views of the key buffers.
     `block_means`: per layer the block sizes (in tokens) whose mean key and mean value are kept next to the rows.  The mean of a
     block is cut into pieces (`mean_piece` elements) and piece i lies at the slot of the block's token i, so the buffers are
-    [N + page, Hkv, piece] -- about 1 / block of the rows' memory -- and a block's mean is handed out and given back with its
+    [Hkv, N + page, piece] -- about 1 / block of the rows' memory -- and a block's mean is handed out and given back with its
     tokens' slots."""
 
     def __init__(self, size: int, page_size: int, dtype: torch.dtype, head_num, head_dim,
@@ -231,7 +231,7 @@ class MHATokenToKVPool:
     def mean_shapes(self, layer_id: int):
         """[(block size, shape of the key means, shape of the value means)] of a layer."""
         rows, h = self.size + self.page_size, self.head_nums[layer_id]
-        return [(p, (rows, h, mean_piece(self.head_dims[layer_id], p)), (rows, h, mean_piece(self.v_head_dims[layer_id], p)))
+        return [(p, (h, rows, mean_piece(self.head_dims[layer_id], p)), (h, rows, mean_piece(self.v_head_dims[layer_id], p)))
                 for p in self.block_sizes[layer_id]]
 
     def _create_buffers(self):

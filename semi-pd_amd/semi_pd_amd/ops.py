@@ -2064,14 +2064,14 @@ def _check_angles(name: str, table: Optional[torch.Tensor], T: int, half: int) -
 
 
 def _check_means(name: str, means, k_buffer: torch.Tensor, v_buffer: torch.Tensor) -> None:
-    """means: (tokens of a block, key means [N, G, piece], value means [N, G, piece]) or None."""
+    """means: (tokens of a block, key means [G, N, piece], value means [G, N, piece]) or None."""
     if means is None:
         return
     pool, km, vm = means
     for m, buf in ((km, k_buffer), (vm, v_buffer)):
-        if m.dim() != 3 or m.shape[:2] != buf.shape[:2] or m.dtype != buf.dtype or not m.is_contiguous() \
+        if m.dim() != 3 or m.shape[:2] != (buf.shape[1], buf.shape[0]) or m.dtype != buf.dtype or not m.is_contiguous() \
                 or m.shape[2] * pool < buf.shape[2]:
-            raise RuntimeError(f"{name}: block means are contiguous [N, G, piece] buffers next to the pools, piece * block >= head size")
+            raise RuntimeError(f"{name}: block means are contiguous [G, N, piece] buffers next to the pools, piece * block >= head size")
 
 
 def head_norm_rope_kv_store(qkv: torch.Tensor, num_q_heads: int, num_kv_heads: int, qk_dim: int, v_dim: int, k_off: int, v_off: int,
@@ -2113,7 +2113,7 @@ def head_norm_rope_kv_store(qkv: torch.Tensor, num_q_heads: int, num_kv_heads: i
     check(_lib.load().semipd_head_norm_rope_kv_store(
         ptr(qkv), qkv.stride(0), T, num_q_heads, num_kv_heads, qk_dim, v_dim, int(k_off), int(v_off), ptr(q_weight), ptr(k_weight),
         float(eps), ptr(qk_angles) if rot_dims else None, int(rot_dims), ptr(v_angles), ptr(k_buffer), ptr(v_buffer), ptr(loc),
-        ptr(positions) if pool else None, int(pool), ptr(km), ptr(vm), km.shape[2] if pool else 0, vm.shape[2] if pool else 0,
+        ptr(positions) if pool else None, int(pool), ptr(km), ptr(vm), km.shape[1] if pool else 0, km.shape[2] if pool else 0, vm.shape[2] if pool else 0,
         ptr(req_to_token) if pool else None, req_to_token.stride(0) if pool else 0, ptr(req_pool_indices) if pool else None,
         ptr(seq_lens) if pool else None, ptr(q_start) if pool else None, ptr(q_len) if pool else None, B, dtype_code(qkv.dtype),
         current_stream(qkv.device)), name)
@@ -2130,7 +2130,7 @@ def block_means(k_buffer: torch.Tensor, v_buffer: torch.Tensor, means, req_to_to
     if req_to_token.dtype != torch.int32 or req_pool_indices.dtype != torch.int64 or seq_lens.dtype != torch.int64:
         raise RuntimeError("block_means: req_to_token int32, req_pool_indices / seq_lens int64")
     check(_lib.load().semipd_block_means(ptr(k_buffer), ptr(v_buffer), k_buffer.shape[1], k_buffer.shape[2], v_buffer.shape[2], int(pool),
-                                         ptr(km), ptr(vm), km.shape[2], vm.shape[2], ptr(req_to_token), req_to_token.stride(0),
+                                         ptr(km), ptr(vm), km.shape[1], km.shape[2], vm.shape[2], ptr(req_to_token), req_to_token.stride(0),
                                          ptr(req_pool_indices), ptr(seq_lens), ptr(q_start), ptr(q_len), B, int(num_tokens),
                                          dtype_code(k_buffer.dtype), current_stream(k_buffer.device)), "block_means")
 
@@ -2169,7 +2169,7 @@ def pooled_window_attention_fwd(q: torch.Tensor, out: torch.Tensor, k_buffer: to
     pool, km, vm = means if means is not None else (0, None, None)
     check(_lib.load().semipd_pooled_window_attention(
         ptr(q), q.stride(0), ptr(gate), gate.stride(0) if gate is not None else 0, ptr(out), out.stride(0), ptr(k_buffer), ptr(v_buffer),
-        ptr(km), ptr(vm), km.shape[2] if pool else 0, vm.shape[2] if pool else 0, ptr(req_to_token), req_to_token.stride(0),
+        ptr(km), ptr(vm), km.shape[1] if pool else 0, km.shape[2] if pool else 0, vm.shape[2] if pool else 0, ptr(req_to_token), req_to_token.stride(0),
         ptr(req_pool_indices), ptr(seq_lens), ptr(q_start), ptr(q_len), B, T, int(max_q_len), H, G, D, E, float(sm_scale), int(window),
         int(pool), ptr(sink), ptr(turn), n_splits, ptr(partial), int(form), dtype_code(q.dtype), current_stream(q.device)), name)
 
@@ -2205,11 +2205,10 @@ def matrix_memory(proj: torch.Tensor, offsets, num_heads: int, qk_dim: int, v_di
         raise RuntimeError("matrix_memory: state_indices / seq_lens are int64 [B]")
     _batch_rows("matrix_memory", T, B, q_start, q_len)
     lib = _lib.load()
-    wld = int(lib.semipd_matrix_memory_work_width(num_heads, v_dim))
-    work = torch.empty((T, wld), dtype=torch.float32, device=proj.device)
+    work = torch.empty(int(lib.semipd_matrix_memory_workspace(T, num_heads, v_dim)), dtype=torch.float32, device=proj.device)
     out = torch.empty((T, inner), dtype=proj.dtype, device=proj.device)
     check(lib.semipd_matrix_memory(ptr(proj), proj.stride(0), q_off, k_off, v_off, g_off, i_off, f_off, ptr(i_bias), ptr(f_bias),
-                                   float(gate_cap), ptr(norm_weight), float(eps), ptr(work), wld, ptr(state), state.stride(0),
+                                   float(gate_cap), ptr(norm_weight), float(eps), ptr(work), work.numel(), ptr(state), state.stride(0),
                                    ptr(state_indices), ptr(seq_lens), ptr(q_start), ptr(q_len), B, T, num_heads, qk_dim, v_dim,
                                    float(qk_dim) ** -0.5, ptr(out), out.stride(0), int(form), dtype_code(proj.dtype),
                                    current_stream(proj.device)), "matrix_memory")

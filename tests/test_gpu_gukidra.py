@@ -85,8 +85,8 @@ def test_head_norms_rotation_store_and_block_means(dtype, H, G, D, E, rot, pool)
     table[0, :61], table[2, :33] = perm[:61].int(), perm[61:94].int()
     table_d = table.to(DEV)
     kp, vp = torch.full((N + 1, G, D), 3.0, dtype=dtype, device=DEV), torch.full((N + 1, G, E), 3.0, dtype=dtype, device=DEV)
-    km = torch.full((N + 1, G, mean_piece(D, pool)), 5.0, dtype=dtype, device=DEV)
-    vm = torch.full((N + 1, G, mean_piece(E, pool)), 5.0, dtype=dtype, device=DEV)
+    km = torch.full((G, N + 1, mean_piece(D, pool)), 5.0, dtype=dtype, device=DEV)
+    vm = torch.full((G, N + 1, mean_piece(E, pool)), 5.0, dtype=dtype, device=DEV)
 
     def run(parts, decode=False):
         x = torch.cat([raw[r][lo:hi] for r, lo, hi in parts]).to(DEV)
@@ -120,24 +120,23 @@ def test_head_norms_rotation_store_and_block_means(dtype, H, G, D, E, rot, pool)
         for cache, means, size in ((kp_c[s], km_c, D), (vp_c[s], vm_c, E)):
             piece, mean = means.shape[2], O.block_means(cache.float(), pool)
             for b in range(n // pool):
-                pieces = means[s[b * pool: (b + 1) * pool]]                     # [pool, G, piece]
-                got = pieces.transpose(0, 1).reshape(G, pool * piece)[:, :size]
+                got = means[:, s[b * pool: (b + 1) * pool]].reshape(G, pool * piece)[:, :size]
                 torch.testing.assert_close(got.float(), mean[b], rtol=2 ** -8 if dtype == torch.bfloat16 else 1e-5, atol=1e-6)
             for tok in range(n // pool * pool, n):                              # a block that is not whole has no mean yet
-                assert (means[s[tok]] == 5.0).all()
+                assert (means[:, s[tok]] == 5.0).all()
     free = [i for i in range(N + 1) if i not in used]
-    assert (kp_c[free] == 3.0).all() and (vp_c[free] == 3.0).all() and (km_c[free] == 5.0).all() and (vm_c[free] == 5.0).all()
+    assert (kp_c[free] == 3.0).all() and (vp_c[free] == 3.0).all() and (km_c[:, free] == 5.0).all() and (vm_c[:, free] == 5.0).all()
     # means of another block size of the same rows, as a second reader of the cache asks for
     other = pool + 1
-    km2 = torch.zeros((N + 1, G, mean_piece(D, other)), dtype=dtype, device=DEV)
-    vm2 = torch.zeros((N + 1, G, mean_piece(E, other)), dtype=dtype, device=DEV)
+    km2 = torch.zeros((G, N + 1, mean_piece(D, other)), dtype=dtype, device=DEV)
+    vm2 = torch.zeros((G, N + 1, mean_piece(E, other)), dtype=dtype, device=DEV)
     rows, lengths, start, n = _batch([(2, 0, 33), (0, 0, 61)])
     ops.block_means(kp, vp, (other, km2, vm2), table_d, rows, lengths, start, n, 94)
     for r, n_ in lens.items():
         s = table[r, :n_].long()
         mean = O.block_means(vp_c[s].float(), other)
         for b in range(n_ // other):
-            got = vm2.cpu()[s[b * other: (b + 1) * other]].transpose(0, 1).reshape(G, -1)[:, :E]
+            got = vm2.cpu()[:, s[b * other: (b + 1) * other]].reshape(G, -1)[:, :E]
             torch.testing.assert_close(got.float(), mean[b], rtol=2 ** -8 if dtype == torch.bfloat16 else 1e-5, atol=1e-6)
 
 
@@ -190,7 +189,7 @@ def test_window_with_pooled_blocks(dtype, form, H, G, D, E, window, pool):
     sink = torch.zeros(H, device=DEV)
     means = None
     if pool:
-        km, vm = (torch.zeros(N + 1, G, mean_piece(d, pool), dtype=dtype, device=DEV) for d in (D, E))
+        km, vm = (torch.zeros(G, N + 1, mean_piece(d, pool), dtype=dtype, device=DEV) for d in (D, E))
         means = (pool, km, vm)
         rows, lens, start, n = _batch([(1, 0, T), (0, 0, other)])
         ops.block_means(kp, vp, means, table, rows, lens, start, n, T + other)

@@ -104,8 +104,8 @@ def test_pool_with_block_means_next_to_the_rows():
     pool = MHATokenToKVPool(10, 1, torch.float32, [2, 1], [12, 64], 2, "cpu", v_head_dim=[8, 40], block_means=[[4, 3], [2]])
     assert not pool.uniform and pool.block_sizes == [[3, 4], [2]]
     block, km, vm = pool.get_block_means(1, 2)
-    assert block == 2 and km.shape == (11, 1, 32) and vm.shape == (11, 1, 32) and pool.get_block_means(0, 0) is None
-    assert pool.get_block_means(0, 4)[1].shape == (11, 2, 8) and pool.get_block_means(0, 3)[2].shape == (11, 2, 8)
+    assert block == 2 and km.shape == (1, 11, 32) and vm.shape == (1, 11, 32) and pool.get_block_means(0, 0) is None
+    assert pool.get_block_means(0, 4)[1].shape == (2, 11, 8) and pool.get_block_means(0, 3)[2].shape == (2, 11, 8)
     # every buffer lies in the one slab and none overlaps another
     bufs = pool.k_buffer + pool.v_buffer + [m for layer in pool.means for pair in layer.values() for m in pair]
     spans = sorted((t.data_ptr(), t.data_ptr() + t.numel() * 4) for t in bufs)

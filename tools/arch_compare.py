@@ -811,8 +811,8 @@ def _gukidra_kernel_pairs(s, tb, dev):
     n_slots = max(T, B2 * C) + 1
     kp = torch.randn(n_slots, G, D, device=dev, dtype=dt)
     vp = torch.randn(n_slots, G, E, device=dev, dtype=dt)
-    km = torch.randn(n_slots, G, mean_piece(D, P), device=dev, dtype=dt)
-    vm = torch.randn(n_slots, G, mean_piece(E, P), device=dev, dtype=dt)
+    km = torch.randn(G, n_slots, mean_piece(D, P), device=dev, dtype=dt)
+    vm = torch.randn(G, n_slots, mean_piece(E, P), device=dev, dtype=dt)
     means = (P, km, vm)
     nw = torch.ones(D, device=dev, dtype=dt)
     freq = 10000.0 ** (-2.0 * torch.arange(D // 2, dtype=torch.float32, device=dev) / D)
@@ -854,7 +854,7 @@ def _gukidra_kernel_pairs(s, tb, dev):
     gate2 = torch.randn(B2, H, device=dev, dtype=dt)
     tab2 = ops.angle_table(torch.full((B2,), C - 1, device=dev, dtype=torch.int64), freq)
     nb = max(0, C - N) // P
-    splits = max(1, min(16, 512 // (B2 * G * ((H // G + 15) // 16)), (N + nb) // 128))       # HipAttnBackend.forward_pooled_window's rule on 256 CUs
+    splits = max(1, min(16, 256 // (B2 * G * ((H // G + 15) // 16)), (N + nb) // 128))       # HipAttnBackend.forward_pooled_window's rule on 256 CUs
     t_new = _timed(lambda: ops.pooled_window_attention_fwd(q2, o2, kp, vp, means, r2t2, rows2, lens2, None, None, 1, D ** -0.5, N, sink=sink,
                                                            gate=gate2, turn=tab2, n_splits=splits))
     t_old = _timed(lambda: ops.window_attention_fwd(q2, o2, kp, vp, r2t2, rows2, lens2, None, None, 1, D ** -0.5, N, 0, None, False, sink))
@@ -868,7 +868,8 @@ def _gukidra_kernel_pairs(s, tb, dev):
     width = sum(sizes) + -sum(sizes) % 8
     ib, fb = torch.zeros(MH, device=dev), torch.zeros(MH, device=dev) + 4.0
     mnw = torch.ones(MH * ME, device=dev, dtype=dt)
-    S = torch.zeros(B2 + 1, ops.matrix_memory_state_width(MH, MD, ME), device=dev)
+    SW = ops.matrix_memory_state_width(MH, MD, ME)
+    S = torch.zeros(B2 + 1, -(-SW // 4) * 4, device=dev)[:, :SW]             # rows on 16-byte boundaries, as in the state pool
     mp = torch.randn(T, width, device=dev, dtype=dt)
     t_new = _timed(lambda: ops.matrix_memory(mp, offs, MH, MD, ME, ib, fb, 15.0, mnw, 1e-5, S, st4, lens, q_start, q_len), iters=10, warm=2)
     SH, SE, SN, SG, taps = tb["sheads"], tb["svdim"], tb["state"], tb["groups"], 4
