@@ -189,8 +189,10 @@ __global__ void __launch_bounds__(256) head_norm_rope_kv_store_vec_kernel(HeadPr
     }
     const int sh = is_v ? a.v_sh : a.k_sh, mask = (1 << sh) - 1;
     T* means = (T*)(is_v ? a.vb_pool : a.kb_pool) + ((head * a.mean_slots) << sh);
-    store16(means + ((int64_t)slots[e0 >> sh] << sh) + (e0 & mask), ox);
-    store16(means + ((int64_t)slots[e1 >> sh] << sh) + (e1 & mask), oy);
+    // (the last token's slot is the row's own: a padded row of a captured batch points at the dummy slot, whatever its table row says)
+    auto slot_of = [&](int i) -> int64_t { return i + 1 < a.pool ? (int64_t)slots[i] : a.loc[t]; };
+    store16(means + (slot_of(e0 >> sh) << sh) + (e0 & mask), ox);
+    store16(means + (slot_of(e1 >> sh) << sh) + (e1 & mask), oy);
   }
 }
 

@@ -725,8 +725,11 @@ template <typename T> struct TokenRows {
   struct Step {
     const TokenRows& r; int64_t j_end;
     __device__ __forceinline__ bool have(int64_t j) const { return j <= j_end; }
-    __device__ __forceinline__ const T* k(int64_t j, int e) const { return r.kp + r.slot(j) * r.kstride + e; }
-    __device__ __forceinline__ const T* v(int64_t j, int e) const { return r.vp + r.slot(j) * r.vstride + e; }
+    // the slot that holds element e of key j, and element e of that slot's row
+    __device__ __forceinline__ int k_slot(int64_t j, int) const { return (int)r.slot(j); }
+    __device__ __forceinline__ int v_slot(int64_t j, int) const { return (int)r.slot(j); }
+    __device__ __forceinline__ const T* k(int slot, int e) const { return r.kp + (int64_t)slot * r.kstride + e; }
+    __device__ __forceinline__ const T* v(int slot, int e) const { return r.vp + (int64_t)slot * r.vstride + e; }
     // a lane's K row: looked up once for all of its pieces (a key that is not there: the dummy slot)
     __device__ __forceinline__ KRow krow(int64_t j) const { return KRow{r.kp + (j <= j_end ? r.slot(j) : 0) * r.kstride}; }
   };
@@ -760,12 +763,10 @@ template <typename T> struct PooledRows {
       }
     };
     __device__ __forceinline__ bool have(int64_t j) const { return (int)j <= last; }
-    __device__ __forceinline__ const T* k(int64_t j, int e) const {
-      return kp + slot((int)j * mul + add + (e >> k_sh)) * kld + (e & k_mask);
-    }
-    __device__ __forceinline__ const T* v(int64_t j, int e) const {
-      return vp + slot((int)j * mul + add + (e >> v_sh)) * vld + (e & v_mask);
-    }
+    __device__ __forceinline__ int k_slot(int64_t j, int e) const { return (int)slot((int)j * mul + add + (e >> k_sh)); }
+    __device__ __forceinline__ int v_slot(int64_t j, int e) const { return (int)slot((int)j * mul + add + (e >> v_sh)); }
+    __device__ __forceinline__ const T* k(int s, int e) const { return kp + (int64_t)s * kld + (e & k_mask); }
+    __device__ __forceinline__ const T* v(int s, int e) const { return vp + (int64_t)s * vld + (e & v_mask); }
     __device__ __forceinline__ KRow krow(int64_t j) const {
       const bool there = (int)j <= last;
       const int pos = (int)j * mul + add;
@@ -785,7 +786,8 @@ template <typename T> struct PooledRows {
 
 // The walk over keys j_begin, j_begin + j_step, ... (steps of 32 keys, keys past j_end masked) for the 16 columns of this wave.
 //   NT threads (a workgroup with BLOCK_SYNC, else one wave) stage the V tile of every step; `tid` is the thread's index among
-//   them.  relevant(j0): whether this wave has anything to multiply in the step at j0 (it stages and syncs anyway).
+//   them.  relevant(j0): 0 if this wave has nothing to multiply in the step at j0 (it stages and syncs anyway), 2 if every one of its
+//   columns sees all 32 keys (nothing is masked), else 1; the same for all lanes of the wave.
 //   ok(j): whether key j is visible to this lane's column.
 //   BLOCK_SYNC (a workgroup walks together): the K rows of a step go through an LDS tile as well, loaded once for all waves
 //   in whole rows; a wave on its own takes its K fragments straight from the pool into operand layout.
@@ -804,8 +806,8 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
   // and one barrier per step separates them
   const int tile_pair = KS * (rs + rsk);
   uint8_t* k_lds = v_lds + KS * rs;
-  uint4 vr[NV];
-  uint4 kr[NK];
+  u32x4 vr[NV];
+  u32x4 kr[NK];
   const ScoreMap smap(scale, cap);
   // which row and which 16 bytes of it each of this thread's pieces is (the same in every step)
   int v_key[NV], v_ec[NV], k_key[NK], k_ec[NK];
@@ -830,23 +832,46 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
       __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
     }
   };
+  // A workgroup looks the slots of a step up one step before it asks for the rows: the loads of the rows wait for nothing.
+  int v_slot[BLOCK_SYNC ? NV : 1], k_slot[NK];
+  auto load_slots = [&](int64_t j0) {
+    if constexpr (BLOCK_SYNC) {
+      const auto at = rows.step(j0, j_end);
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int64_t j = j0 + v_key[i];
+        if (v_key[i] >= 0 && at.have(j)) v_slot[i] = at.v_slot(j, v_ec[i] * 8);
+      }
+#pragma unroll
+      for (int i = 0; i < NK; ++i) {
+        const int64_t j = j0 + k_key[i];
+        if (k_key[i] >= 0 && at.have(j)) k_slot[i] = at.k_slot(j, k_ec[i] * 8);
+      }
+    }
+  };
   auto load_v = [&](int64_t j0) {
     const auto at = rows.step(j0, j_end);
 #pragma unroll
     for (int i = 0; i < NV; ++i)
       if (v_key[i] >= 0) {
         const int64_t j = j0 + v_key[i];
-        vr[i] = at.have(j) ? *reinterpret_cast<const uint4*>(at.v(j, v_ec[i] * 8)) : uint4{0u, 0u, 0u, 0u};
+        vr[i] = u32x4{0u, 0u, 0u, 0u};
+        if (at.have(j)) {
+          int slot;
+          if constexpr (BLOCK_SYNC) slot = v_slot[i];
+          else slot = at.v_slot(j, v_ec[i] * 8);
+          vr[i] = *reinterpret_cast<const u32x4*>(at.v(slot, v_ec[i] * 8));
+        }
       }
   };
   auto store_v = [&](int buf) {        // buf: which pair of tiles (a lone wave has one)
 #pragma unroll
     for (int i = 0; i < NV; ++i)
-      if (v_key[i] >= 0) *reinterpret_cast<uint4*>(v_lds + buf * tile_pair + v_key[i] * rs + v_ec[i] * 16) = vr[i];
+      if (v_key[i] >= 0) *reinterpret_cast<u32x4*>(v_lds + buf * tile_pair + v_key[i] * rs + v_ec[i] * 16) = vr[i];
     if constexpr (BLOCK_SYNC) {
 #pragma unroll
       for (int i = 0; i < NK; ++i)
-        if (k_key[i] >= 0) *reinterpret_cast<uint4*>(k_lds + buf * tile_pair + k_key[i] * rsk + k_ec[i] * 16) = kr[i];
+        if (k_key[i] >= 0) *reinterpret_cast<u32x4*>(k_lds + buf * tile_pair + k_key[i] * rsk + k_ec[i] * 16) = kr[i];
     }
   };
   auto load_k_rows = [&](int64_t j0) {
@@ -855,7 +880,8 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
     for (int i = 0; i < NK; ++i)
       if (k_key[i] >= 0) {
         const int64_t j = j0 + k_key[i];
-        kr[i] = at.have(j) ? *reinterpret_cast<const uint4*>(at.k(j, k_ec[i] * 8)) : uint4{0u, 0u, 0u, 0u};
+        kr[i] = u32x4{0u, 0u, 0u, 0u};
+        if (at.have(j)) kr[i] = *reinterpret_cast<const u32x4*>(at.k(k_slot[i], k_ec[i] * 8));
       }
   };
   auto load_k = [&](int64_t j0, auto& k) {
@@ -869,7 +895,7 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
         k.b[kk].u = *reinterpret_cast<const uint4*>(pb.at(8 * g + 32 * kk));
       }
   };
-  auto compute = [&](int64_t j0, const auto& k, int half, auto after_scores) {   // keys j0 .. j0 + 31 out of tile pair `half`
+  auto compute = [&](int64_t j0, const auto& k, int half, bool masked, auto after_scores) {   // keys j0 .. j0 + 31 out of tile pair `half`
     f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = {0.f, 0.f, 0.f, 0.f};
     if constexpr (BLOCK_SYNC) {
       const uint8_t* ra = k_lds + half * tile_pair + r * rsk + g * 16;
@@ -896,8 +922,15 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
     const int64_t ja = j0 + 4 * g, jb = ja + 16;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      sc[i] = ok(ja + i) ? smap(sa[i]) : -INFINITY;
-      sc[4 + i] = ok(jb + i) ? smap(sb[i]) : -INFINITY;
+      sc[i] = smap(sa[i]);
+      sc[4 + i] = smap(sb[i]);
+    }
+    if (masked) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        sc[i] = ok(ja + i) ? sc[i] : -INFINITY;
+        sc[4 + i] = ok(jb + i) ? sc[4 + i] : -INFINITY;
+      }
     }
     float p[8];
     if constexpr (SIG) {
@@ -948,10 +981,12 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
   };
   if (j_begin > j_end) return;
   KFrags<BLOCK_SYNC ? 1 : ND> k0;      // one set: a lone wave refills it as soon as the scores of a step are taken
+  load_slots(j_begin);
   load_v(j_begin);
   if constexpr (BLOCK_SYNC) load_k_rows(j_begin);
   else load_k(j_begin, k0);
   if constexpr (BLOCK_SYNC) {
+    if (j_begin + j_step <= j_end) load_slots(j_begin + j_step);
     store_v(0);
     sync();
     int buf = 0;
@@ -960,8 +995,10 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
       if (jn <= j_end) {                                 // in flight while this step is multiplied
         load_v(jn);
         load_k_rows(jn);
+        if (jn + j_step <= j_end) load_slots(jn + j_step);
       }
-      if (relevant(j0)) compute(j0, k0, buf, [] {});
+      const int what = relevant(j0);
+      if (what) compute(j0, k0, buf, what != 2, [] {});
       if (jn <= j_end) store_v(buf ^ 1);
       sync();       // the next step's rows are in place, and everyone is done with this step's
     }
@@ -972,7 +1009,7 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
       store_v(0);
       sync();
       if (jn <= j_end) load_v(jn);                       // in flight while this step is multiplied
-      compute(j0, k0, 0, [&] {
+      compute(j0, k0, 0, relevant(j0) != 2, [&] {
         if (jn <= j_end) load_k(jn, k0);
       });
     }
@@ -981,7 +1018,7 @@ __device__ __forceinline__ void key_walk(SoftState<NE>& st, const Frag16 (&qf)[N
 
 // Prompt portions: 64 query rows of one request and one head per workgroup, 16 per wave.
 template <typename T, int ND, int NE, bool SIG, bool POOL>
-__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 4 ? 4 : 1))) local_attention_mfma_kernel(LocalAttnArgs a) {
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 2 ? 4 : (ND <= 4 ? 3 : 1)))) local_attention_mfma_kernel(LocalAttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) uint8_t v_lds[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
   // Workgroup -> (kv head, 64-row tile, q head of the group), the last fastest.  Consecutive workgroup ids go round the
@@ -1055,26 +1092,36 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(ND <= 
     const int64_t my_nb = blocks_seen(a, my_pos), w_nb = blocks_seen(a, w_hi);
     const PooledRows<T> prows{rows, false, (const T*)a.kb_pool + ((gk * a.mean_slots) << a.k_sh),
                               (const T*)a.vb_pool + ((gk * a.mean_slots) << a.v_sh), a.k_sh, a.v_sh, a.pool, nb, nb_pad, blk_lo};
+    const int pad = (int)nb_pad, mine = q_ok ? (int)my_nb : 0, to = q_ok ? (int)(my_pos - blk_lo) + pad : -1, from = (int)(my_lo - blk_lo) + pad;
+    const int w_first = __builtin_amdgcn_readfirstlane((int)(base_pos + wq0 - blk_lo) + pad);      // the wave's first row, as a key
+    const int w_last = __builtin_amdgcn_readfirstlane((int)(w_hi - blk_lo) + pad);
+    const int w_from = __builtin_amdgcn_readfirstlane((int)(w_lo - blk_lo) + pad);                 // where the first row's window starts,
+    const int w_full = __builtin_amdgcn_readfirstlane((int)(lo_of(w_hi) - blk_lo) + pad);          // the last row's
+    const int w_seen = __builtin_amdgcn_readfirstlane((int)w_nb);
+    const int w_all = __builtin_amdgcn_readfirstlane((int)blocks_seen(a, base_pos + wq0));
     key_walk<T, ND, NE, 256, true, false>(
         st, qf, nd, ne, E, prows, 0, nb_pad + blk_hi - blk_lo, 32, v_lds, tid, a.scale, a.cap,
-        [&](int64_t j) {
-          const int64_t p = blk_lo + j - nb_pad;
-          return q_ok && (j < nb_pad ? j < my_nb : (p <= my_pos && p >= my_lo));
-        },
+        [&](int64_t j) { return (int)j < pad ? (int)j < mine : ((int)j <= to && (int)j >= from); },
         [&](int64_t j0) {
-          const int64_t p = blk_lo + j0 - nb_pad;
-          return wave_on && (j0 < nb_pad ? j0 < w_nb : (p <= w_hi && p + 31 >= w_lo));
+          const int j = (int)j0;
+          if (!wave_on) return 0;
+          if (j < pad) return j >= w_seen ? 0 : (j + 31 < w_all ? 2 : 1);
+          return (j > w_last || j + 31 < w_from) ? 0 : ((j + 31 <= w_first && j >= w_full) ? 2 : 1);
         }, r, g);
   } else {
     // the kept first positions that lie in front of the tile's window range: visible to every row of the tile
     const int64_t n_first = keep < blk_lo ? keep : blk_lo;
     if (n_first > 0)
       key_walk<T, ND, NE, 256, true, SIG>(st, qf, nd, ne, E, rows, 0, n_first - 1, 32, v_lds, tid, a.scale, a.cap,
-                                          [&](int64_t j) { return q_ok && j < n_first; }, [&](int64_t) { return wave_on; }, r, g, hb);
+                                          [&](int64_t j) { return q_ok && j < n_first; }, [&](int64_t) { return wave_on ? 1 : 0; }, r, g, hb);
+    const int64_t w_first = base_pos + wq0, w_full = lo_of(w_hi);
     key_walk<T, ND, NE, 256, true, SIG>(
         st, qf, nd, ne, E, rows, blk_lo, blk_hi, 32, v_lds, tid, a.scale, a.cap,
         [&](int64_t j) { return q_ok && j <= my_pos && (j >= my_lo || j < keep); },
-        [&](int64_t j0) { return wave_on && j0 <= w_hi && (j0 + 31 >= w_lo || j0 < keep); }, r, g, hb);
+        [&](int64_t j0) {
+          if (!(wave_on && j0 <= w_hi && (j0 + 31 >= w_lo || j0 < keep))) return 0;
+          return __builtin_amdgcn_readfirstlane((int)(j0 + 31 <= w_first && j0 >= w_full)) ? 2 : 1;
+        }, r, g, hb);
   }
   float l = st.l;
   l += __shfl_xor(l, 16, 64);
@@ -1253,16 +1300,19 @@ __global__ void __launch_bounds__(64 * NW) local_attention_decode_kernel(LocalAt
                               (const T*)a.vb_pool + ((gk * a.mean_slots) << a.v_sh), a.k_sh, a.v_sh, a.pool, nb, nb_pad, lo_q};
     key_walk<T, ND, NE, 64, false, false>(st, qf, nd, ne, E, prows, lo + 32 * wave, pos, 32 * NW, mine_b, lane, a.scale, a.cap,
                                           [&](int64_t j) { return j < nb_pad ? j < nb && j <= pos : j <= pos; },
-                                          [&](int64_t) { return true; }, r, g);
+                                          [&](int64_t j0) {
+                                            return __builtin_amdgcn_readfirstlane((int)(j0 + 31 < (j0 < nb_pad ? nb : pos + 1))) ? 2 : 1;
+                                          }, r, g);
   } else {
     // the kept first positions in front of the window (none without one), then the range that ends at the query
     if (n_first > 0) {
       const TokenRows<T> first{rows.kp, rows.kstride, rows.vp, rows.vstride, row, nullptr, 0};
       key_walk<T, ND, NE, 64, false, SIG>(st, qf, nd, ne, E, first, (int64_t)32 * wave, n_first - 1, 32 * NW, mine_b, lane, a.scale,
-                                          a.cap, [&](int64_t j) { return j < n_first; }, [&](int64_t) { return true; }, r, g, hb);
+                                          a.cap, [&](int64_t j) { return j < n_first; }, [&](int64_t) { return 1; }, r, g, hb);
     }
     key_walk<T, ND, NE, 64, false, SIG>(st, qf, nd, ne, E, rows, lo + 32 * wave, pos, 32 * NW, mine_b, lane, a.scale, a.cap,
-                                        [&](int64_t j) { return j <= pos; }, [&](int64_t) { return true; }, r, g, hb);
+                                        [&](int64_t j) { return j <= pos; },
+                                        [&](int64_t j0) { return __builtin_amdgcn_readfirstlane((int)(j0 + 31 <= pos)) ? 2 : 1; }, r, g, hb);
   }
   float l = st.l;
   l += __shfl_xor(l, 16, 64);
@@ -1539,7 +1589,7 @@ static int launch_attention(LocalAttnArgs a, int64_t max_q_len, int form, int dt
     size_t tiles = 2 * ((size_t)tile + 32 * (size_t)(qk_dim * 2 + 32));   // two pairs of (32 V rows, 32 K rows): at most 71.7 KB
     const size_t epilogue = 4 * 16 * (size_t)(v_dim + 4) * sizeof(float);       // POOL: the result in fp32
     if (POOL && epilogue > tiles) tiles = epilogue;
-    static std::atomic<uint64_t> done_p[8] = {};
+    static std::atomic<uint64_t> done_p[12] = {};
 #define SEMIPD_LA_PRE(TT, NDD, NEE, SS, SLOT)                                                                                   \
   do {                                                                                                                          \
     if (tiles > 65536 && ensure_dynamic_lds((const void*)local_attention_mfma_kernel<TT, NDD, NEE, SS && !POOL, POOL>, kMaxDynLds, done_p[SLOT], \
@@ -1547,7 +1597,14 @@ static int launch_attention(LocalAttnArgs a, int64_t max_q_len, int form, int dt
       return SEMIPD_EINVAL;                                                                                                     \
     hipLaunchKernelGGL((local_attention_mfma_kernel<TT, NDD, NEE, SS && !POOL, POOL>), grid, dim3(256), tiles, as_stream(stream), a);           \
   } while (0)
-    if (dtype == SEMIPD_BF16) {
+    const bool tiny = qk_dim <= 64 && v_dim <= 64;      // half the operand registers: nothing of the walk leaves them
+    if (tiny && dtype == SEMIPD_BF16) {
+      if (!sig) SEMIPD_LA_PRE(bf16_t, 2, 4, false, 8);
+      else SEMIPD_LA_PRE(bf16_t, 2, 4, true, 9);
+    } else if (tiny) {
+      if (!sig) SEMIPD_LA_PRE(f16_t, 2, 4, false, 10);
+      else SEMIPD_LA_PRE(f16_t, 2, 4, true, 11);
+    } else if (dtype == SEMIPD_BF16) {
       if (small && !sig) SEMIPD_LA_PRE(bf16_t, 4, 8, false, 0);
       else if (small) SEMIPD_LA_PRE(bf16_t, 4, 8, true, 1);
       else if (!sig) SEMIPD_LA_PRE(bf16_t, 8, 16, false, 2);

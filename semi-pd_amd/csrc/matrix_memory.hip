@@ -68,7 +68,6 @@ __device__ __forceinline__ bool memory_rows(const MemArgs& a, int b, int64_t& t0
 // ---------------------------------------------------------------------------------- prompt batches on the matrix cores
 constexpr int kMemChunk = 64;       // tokens of a chunk
 constexpr int kMemCols = 32;        // columns of S of a workgroup
-typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 constexpr float kMemLog2e = 1.4426950408889634f;
 
 

@@ -52,6 +52,7 @@ template <> __device__ inline uint32_t pack2<f16_t>(float a, float b) {
 
 // v_mfma_f32_16x16x32 (lane l: r = l & 15, g = l >> 4): a = A[row r][k 8g .. 8g+7], b = B[k 8g .. 8g+7][col r], d[i] = D[row 4g + i][col r]
 typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 
 template <typename T> __device__ __forceinline__ f32x4 mma16(const Frag16& a, const Frag16& b, f32x4 c);
 template <> __device__ __forceinline__ f32x4 mma16<bf16_t>(const Frag16& a, const Frag16& b, f32x4 c) {

@@ -531,6 +531,21 @@ def test_other_sizes_and_orders(name, dtype, tmp_path):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", ["minimal", "attention_only"])
+def test_padded_rows_of_a_decode_graph_leave_the_pools_alone(name, dtype, tmp_path):
+    """Three requests decode through a graph captured for four: the padded row (a sequence of one token, which completes a block
+    where blocks are of one token) must not touch what the request in row 0 of the table holds."""
+    cfg = CONFIGS[name]
+    w = _write_checkpoint(str(tmp_path), cfg, seed=6)
+    sched = _scheduler(str(tmp_path), dtype, max_tokens=256)
+    assert 3 not in sched.model_runner.graph_runner.capture_bs and 4 in sched.model_runner.graph_runner.capture_bs
+    prompts = {n: _tokens(k, cfg["vocab"], i) for i, (n, k) in enumerate((("x", 60), ("y", 45), ("z", 50)))}
+    got = _run_schedule(sched, prompts, [[("x", 30), ("y", 15), ("z", 20)]] + [[("x", 1), ("y", 1), ("z", 1)]] * 30)
+    for n in prompts:
+        assert _rel_err(got[n], O.forward(cfg, w, prompts[n]), dtype != "float32") < LIMIT[dtype], n
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_eager_decode_steps_and_the_plain_kernel_forms(dtype, tmp_path, monkeypatch):
     """Without captured graphs, the attention a wave per row and the memory token by token."""
     monkeypatch.setenv("SEMIPD_LOCAL_ATTN_FORM", "1")
