@@ -1002,10 +1002,10 @@ int semipd_state_space(const void* proj, int64_t ld, int64_t z_off, int64_t x_of
 int semipd_outnorm_stream(const void* y, int64_t y_ld, float* stream, int64_t stream_ld, const void* weight, float weight_shift,
                           float eps, const void* next_weight, float next_shift, float next_eps, void* out, int64_t out_ld,
                           int64_t rows, int64_t width, int dtype, void* stream_handle);
-/* out (fp32 [rows, half, 2]) = (cos, sin) of positions[t] * freq[i] (fp32 product). */
-int semipd_angle_table(const int64_t* positions, const float* freq, int half, int64_t rows, float* out, void* stream);
+/* out (fp32 [rows, half, 2]) = (cos, sin) of positions[t] * freq[i] (fp32 product), times factor. */
+int semipd_angle_table(const int64_t* positions, const float* freq, int half, int64_t rows, float factor, float* out, void* stream);
 /* Rows of qkv hold q | k | v at columns 0, k_off, v_off (num_kv_heads 0: queries only).  Every head of q and k: RMS norm times
- * q_weight / k_weight [qk_dim], the first rot_dims elements turned in pairs (i, i + rot_dims / 2) by qk_angles (rows of
+ * q_weight / k_weight [qk_dim] (both NULL: no norm), the first rot_dims elements turned in pairs (i, i + rot_dims / 2) by qk_angles (rows of
  * semipd_angle_table); every head of v turned over all v_dim elements in pairs (m, m + v_dim / 2) by v_angles (NULL: v passes).
  * q in place, k and v into the pools at loc.  pool > 0: also the mean key and value of every block of `pool` tokens
  * (counted from the start of a sequence) that the batch completes, as semipd_block_means. */
@@ -1050,6 +1050,31 @@ int semipd_matrix_memory(const void* proj, int64_t ld, int64_t q_off, int64_t k_
                          const int64_t* seq_lens, const int32_t* q_start, const int32_t* q_len, int64_t batch, int64_t num_tokens,
                          int num_heads, int qk_dim, int v_dim, float q_scale, void* out, int64_t out_ld, int form, int dtype,
                          void* stream);
+/* stream (fp32 rows, in place) += y + the n_more rows of more [rows, n_more, width] (either may be missing); out (may be NULL)
+ * receives the new stream in `dtype`.  No reference counterpart. */
+int semipd_add_stream(const void* y, int64_t y_ld, const void* more, int n_more, float* stream, int64_t stream_ld, void* out,
+                      int64_t out_ld, int64_t rows, int64_t width, int dtype, void* stream_handle);
+/* out [rows, width] = gelu_tanh(z) * table[ids[row], col .. col + width). */
+int semipd_gelu_mul_rows(const void* z, int64_t z_ld, const int64_t* ids, const void* table, int64_t table_ld, int64_t col, void* out,
+                         int64_t out_ld, int64_t rows, int64_t width, int dtype, void* stream);
+/* Gated activations, act 0 relu / 1 silu: x rows hold `groups` blocks of 2 ff columns, gate at 0 and up at up_off of a block; out
+ * [rows, groups * ff] = act(gate) * up, with routing times the weight of the block's expert for the row (0: not used). */
+int semipd_glu(const void* x, int64_t x_ld, void* out, int64_t out_ld, int64_t rows, int64_t ff, int64_t up_off, int groups,
+               const float* topk_weights, const int32_t* topk_ids, int topk, int act, int dtype, void* stream);
+/* Linear attention with decays behind its projection GEMM: rows [q | k | v | g] at the given columns, S <- diag(alpha) S + k v^T,
+ * o = S^T q * q_scale per head.  alpha: per channel sigmoid(a2 a + a2_bias)^(1 / tau), a [rank] at column a_off, a2 [H * qk_dim,
+ * rank] of the activation type, a2_bias fp32; or (a2 NULL) a constant per head, powers fp32 [H, 65] = its powers 0 .. 64.
+ * qkv_silu: q, k, v through silu.  o: RMS norm over all heads together (norm_w [H * v_dim]) or per head (norm_w [v_dim]), times
+ * sigmoid(g) or silu(g) -> out [T, H * v_dim].  state fp32 [slots, >= H * qk_dim * v_dim] is a column range of the requests'
+ * state rows.  Batch description as in semipd_local_attention.  form: 0 by shape and type, 1 token by token, 2 the matrix-core
+ * form.  _workspace: fp32 elements of `work`; extend: the batch has q_start. */
+int64_t semipd_linear_attention_workspace(int64_t num_tokens, int64_t batch, int num_heads, int qk_dim, int v_dim, int extend, int dtype);
+int semipd_linear_attention(const void* proj, int64_t ld, int64_t q_off, int64_t k_off, int64_t v_off, int64_t g_off, int64_t a_off,
+                            int rank, const void* a2, const float* a2_bias, float tau, const float* powers, int qkv_silu,
+                            const void* norm_w, int norm_together, float eps, int gate_silu, float* work, int64_t work_elems,
+                            float* state, int64_t state_ld, const int64_t* state_indices, const int64_t* seq_lens,
+                            const int32_t* q_start, const int32_t* q_len, int64_t batch, int64_t num_tokens, int num_heads, int qk_dim,
+                            int v_dim, float q_scale, void* out, int64_t out_ld, int form, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

@@ -1,9 +1,9 @@
 // Between the projection GEMM and the attention: angle tables, per-head norms with rotation of queries, keys AND values, pool
 // stores, and the means of whole blocks of cached tokens (gfx950, wave64).
 //
-//  * angle_table_kernel: (cos, sin) of position * freq[i] for every row of a batch, fp32.  Computed once per forward pass for
-//    every distinct set of frequencies; all layers read it.
-//  * head_norm_rope_kv_store_kernel / _vec_kernel: per head q and k to unit RMS times a weight all heads share, the first
+//  * angle_table_kernel: (cos, sin) of position * freq[i], times a factor, for every row of a batch, fp32.  Computed once per
+//    forward pass for every distinct set of frequencies; all layers read it.
+//  * head_norm_rope_kv_store_kernel / _vec_kernel: per head q and k to unit RMS times a weight all heads share (no norm without weights), the first
 //    rot elements turned in pairs (i, i + rot / 2); values turned over the whole head in pairs (m, m + E / 2); q in place,
 //    k and v into the pools.  A layer that reads another layer's cache prepares its queries only (no k / v heads).
 //  * block_means_kernel: the mean key and the mean value of every block of `pool` tokens that the batch completes, as the
@@ -16,20 +16,20 @@
 namespace semipd {
 
 __global__ void __launch_bounds__(256) angle_table_kernel(const int64_t* __restrict__ positions, const float* __restrict__ freq,
-                                                          int half, int64_t rows, float2* __restrict__ out) {
+                                                          int half, int64_t rows, float factor, float2* __restrict__ out) {
   const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (i >= rows * half) return;
   const int64_t t = i / half;
   float sn, cs;
   sincosf((float)positions[t] * freq[i - t * half], &sn, &cs);
-  out[i] = float2{cs, sn};
+  out[i] = float2{cs * factor, sn * factor};
 }
 
 struct HeadPrepArgs {
   void* qkv; int64_t ld; int64_t num_tokens;
   int H, G, D, E;
   int64_t k_off, v_off;
-  const void* q_w; const void* k_w;          // [D] of the activation type
+  const void* q_w; const void* k_w;          // [D] of the activation type, or both NULL: no norm
   float eps;
   const float* qk_cs; int rot;               // [rows, rot / 2] (cos, sin)
   const float* v_cs;                         // [rows, E / 2] (cos, sin) or NULL: values pass
@@ -59,22 +59,25 @@ __global__ void __launch_bounds__(256) head_norm_rope_kv_store_kernel(HeadPrepAr
     T* src = is_q ? row + (int64_t)u * D : row + a.k_off + (int64_t)(u - a.H) * D;
     T* dst = is_q ? src : (T*)a.k_pool + (a.loc[t] * G + (u - a.H)) * D;
     const T* w = (const T*)(is_q ? a.q_w : a.k_w);
-    float ss = 0.f;
-    for (int d = lane; d < D; d += 64) {
-      const float x = Elem<T>::to_f(src[d]);
-      ss += x * x;
+    float rs = 1.0f;
+    if (w) {
+      float ss = 0.f;
+      for (int d = lane; d < D; d += 64) {
+        const float x = Elem<T>::to_f(src[d]);
+        ss += x * x;
+      }
+      rs = 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps);
     }
-    const float rs = 1.0f / sqrtf(wave_sum(ss) / (float)D + a.eps);
+    auto element = [&](int d) { return w ? Elem<T>::to_f(src[d]) * rs * Elem<T>::to_f(w[d]) : Elem<T>::to_f(src[d]); };
     const int half = a.rot >> 1;
     const float2* cs = reinterpret_cast<const float2*>(a.qk_cs) + t * half;
     for (int i = lane; i < half; i += 64) {          // (a pair is read and written by one lane: q in place)
-      const float x = Elem<T>::to_f(src[i]) * rs * Elem<T>::to_f(w[i]);
-      const float y = Elem<T>::to_f(src[i + half]) * rs * Elem<T>::to_f(w[i + half]);
+      const float x = element(i), y = element(i + half);
       const float2 c = cs[i];
       dst[i] = Elem<T>::from_f(x * c.x - y * c.y);
       dst[i + half] = Elem<T>::from_f(y * c.x + x * c.y);
     }
-    for (int d = a.rot + lane; d < D; d += 64) dst[d] = Elem<T>::from_f(Elem<T>::to_f(src[d]) * rs * Elem<T>::to_f(w[d]));
+    for (int d = a.rot + lane; d < D; d += 64) dst[d] = Elem<T>::from_f(element(d));
   } else {
     const int gv = u - a.H - G;
     const T* src = row + a.v_off + (int64_t)gv * E;
@@ -129,9 +132,9 @@ __global__ void __launch_bounds__(256) head_norm_rope_kv_store_vec_kernel(HeadPr
 #pragma unroll
   for (int o = L / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
   if (!mine) return;
-  if (!is_v) {
+  const T* w = (const T*)(is_q ? a.q_w : a.k_w);
+  if (!is_v && w) {
     const float rs = 1.0f / sqrtf(ss / (float)D + a.eps);
-    const T* w = (const T*)(is_q ? a.q_w : a.k_w);
     const Vec16<T> wx = load16(w + e0), wy = load16(w + e1);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
@@ -269,13 +272,13 @@ __global__ void __launch_bounds__(256) block_means_kernel(HeadPrepArgs a) {
 
 using namespace semipd;
 
-extern "C" int semipd_angle_table(const int64_t* positions, const float* freq, int half, int64_t rows, float* out, void* stream) {
+extern "C" int semipd_angle_table(const int64_t* positions, const float* freq, int half, int64_t rows, float factor, float* out, void* stream) {
   SEMIPD_CHECK_ARG(rows >= 0 && half >= 0, SEMIPD_EINVAL, "angle_table: bad sizes");
   if (rows == 0 || half == 0) return 0;
   SEMIPD_CHECK_ARG(positions && freq && out, SEMIPD_EINVAL, "angle_table: null pointer");
   const int64_t n = rows * half;
   hipLaunchKernelGGL(angle_table_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, as_stream(stream), positions, freq, half, rows,
-                     reinterpret_cast<float2*>(out));
+                     factor, reinterpret_cast<float2*>(out));
   return launch_status("angle_table");
 }
 
@@ -322,10 +325,10 @@ extern "C" int semipd_head_norm_rope_kv_store(void* qkv, int64_t ld, int64_t num
   SEMIPD_CHECK_ARG(num_tokens >= 0 && num_q_heads >= 0 && num_kv_heads >= 0 && num_q_heads + num_kv_heads > 0 && qk_dim > 0,
                    SEMIPD_EINVAL, "head_norm_rope_kv_store: bad sizes");
   if (num_tokens == 0) return 0;
-  SEMIPD_CHECK_ARG(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= qk_dim && (num_kv_heads == 0 || (v_dim > 0 && v_dim % 2 == 0)),
+  SEMIPD_CHECK_ARG(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= qk_dim && (num_kv_heads == 0 || (v_dim > 0 && (!v_angles || v_dim % 2 == 0))),
                    SEMIPD_ESHAPE, "head_norm_rope_kv_store: %d turned elements of a head of %d, value heads of %d", rot_dims, qk_dim, v_dim);
-  SEMIPD_CHECK_ARG(qkv && (num_q_heads == 0 || q_weight) && (rot_dims == 0 || qk_angles) &&
-                       (num_kv_heads == 0 || (k_weight && k_pool && v_pool && loc)),
+  SEMIPD_CHECK_ARG(qkv && (num_q_heads == 0 || num_kv_heads == 0 || (q_weight == nullptr) == (k_weight == nullptr)) &&
+                       (rot_dims == 0 || qk_angles) && (num_kv_heads == 0 || (k_pool && v_pool && loc)),
                    SEMIPD_EINVAL, "head_norm_rope_kv_store: null pointer");
   SEMIPD_CHECK_ARG(ld >= (int64_t)num_q_heads * qk_dim &&
                        (num_kv_heads == 0 || (k_off >= (int64_t)num_q_heads * qk_dim && v_off >= k_off + (int64_t)num_kv_heads * qk_dim &&

@@ -535,6 +535,90 @@ __global__ void __launch_bounds__(256) outnorm_stream_kernel(const T* __restrict
     out[r * out_ld + i] = Elem<T>::from_f(x[i] * rs2 * (Elem<T>::to_f(w2[i]) + shift2));
 }
 
+// ---- two sublayers that read the same input: stream <- stream + y + sum_j more[j]  (fp32, in place), the sum in the activation type
+// for the GEMM behind it.  more: `n_more` rows of `width` per row of the stream (a token's weighted experts, unsummed).
+template <typename T, int V>
+__global__ void __launch_bounds__(256) add_stream_kernel(const T* __restrict__ y, int64_t y_ld, const T* __restrict__ more, int n_more,
+                                                         float* __restrict__ stream, int64_t s_ld, T* __restrict__ out, int64_t out_ld,
+                                                         int64_t rows, int64_t width) {
+  const int64_t per = width / V, n = rows * per;
+  for (int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x; id < n; id += (int64_t)gridDim.x * 256) {
+    const int64_t r = id / per, i = (id - r * per) * V;
+    if constexpr (V == 8) {
+      float x[8], f[8];
+      load8f(stream + r * s_ld + i, x);
+      if (y) {
+        load8f(y + r * y_ld + i, f);
+#pragma unroll
+        for (int u = 0; u < 8; ++u) x[u] += f[u];
+      }
+      for (int j = 0; j < n_more; ++j) {
+        load8f(more + (r * n_more + j) * width + i, f);
+#pragma unroll
+        for (int u = 0; u < 8; ++u) x[u] += f[u];
+      }
+      store8f(stream + r * s_ld + i, x);
+      if (out) store8f(out + r * out_ld + i, x);
+    } else {
+      float x = stream[r * s_ld + i];
+      if (y) x += Elem<T>::to_f(y[r * y_ld + i]);
+      for (int j = 0; j < n_more; ++j) x += Elem<T>::to_f(more[(r * n_more + j) * width + i]);
+      stream[r * s_ld + i] = x;
+      if (out) out[r * out_ld + i] = Elem<T>::from_f(x);
+    }
+  }
+}
+
+// ---- out = gelu(z) * table[id]: the tanh form of gelu, a column range of the row of a token's id, fp32 arithmetic
+__device__ __forceinline__ float gelu_tanh_f(float z) {
+  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+template <typename T>
+__global__ void __launch_bounds__(256) gelu_mul_rows_kernel(const T* __restrict__ z, int64_t z_ld, const int64_t* __restrict__ ids,
+                                                            const T* __restrict__ table, int64_t table_ld, int64_t col,
+                                                            T* __restrict__ out, int64_t out_ld, int64_t rows, int64_t width) {
+  const int64_t n = rows * width;
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
+    const int64_t r = i / width, c = i - r * width;
+    out[r * out_ld + c] = Elem<T>::from_f(gelu_tanh_f(Elem<T>::to_f(z[r * z_ld + c])) * Elem<T>::to_f(table[ids[r] * table_ld + col + c]));
+  }
+}
+
+// ---- gated activations over column ranges: out = act(gate) * up, act relu or silu; `groups` blocks [gate ff | up ff] side by side,
+// with routing times the weight of the block's expert for the row (0 where the row does not use it).
+enum { kGluRelu = 0, kGluSilu = 1 };
+__device__ __forceinline__ float glu_f(float a, float b, int act) {
+  return (act == kGluRelu ? fmaxf(a, 0.f) : a / (1.0f + expf(-a))) * b;
+}
+template <typename T, int V>
+__global__ void __launch_bounds__(256) glu_kernel(const T* __restrict__ x, int64_t x_ld, T* __restrict__ out, int64_t out_ld,
+                                                  int64_t rows, int64_t ff, int64_t up_off, int groups,
+                                                  const float* __restrict__ topk_weights, const int32_t* __restrict__ topk_ids, int topk,
+                                                  int act) {
+  const int64_t width = ff * groups, per = width / V, n = rows * per;
+  for (int64_t id = (int64_t)blockIdx.x * 256 + threadIdx.x; id < n; id += (int64_t)gridDim.x * 256) {
+    const int64_t r = id / per, c = (id - r * per) * V;
+    const int64_t e = groups > 1 ? c / ff : 0, f = c - e * ff;
+    float wgt = 1.f;
+    if (topk_ids) {
+      wgt = 0.f;
+      for (int k = 0; k < topk; ++k)
+        if (topk_ids[r * topk + k] == (int)e) wgt = topk_weights[r * topk + k];
+    }
+    const T* row = x + r * x_ld + e * 2 * ff + f;
+    if constexpr (V == 8) {
+      float a[8], b[8];
+      load8f(row, a);
+      load8f(row + up_off, b);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) a[u] = glu_f(a[u], b[u], act) * wgt;
+      store8f(out + r * out_ld + c, a);
+    } else {
+      out[r * out_ld + c] = Elem<T>::from_f(glu_f(Elem<T>::to_f(row[0]), Elem<T>::to_f(row[up_off]), act) * wgt);
+    }
+  }
+}
+
 // The request that owns row t of a batch, the row's index in the request's portion, the portion's length and the position
 // of its first row (q_start == NULL: row t is request t's newest token).
 __device__ __forceinline__ bool portion_of_row(int64_t t, int64_t batch, const int64_t* seq_lens, const int32_t* q_start,
@@ -855,6 +939,63 @@ extern "C" int semipd_outnorm_stream(const void* y, int64_t y_ld, float* stream,
   });
 #undef SEMIPD_OUTNORM
   return launch_status("outnorm_stream");
+}
+
+static unsigned grid_for(int64_t items) {
+  const int64_t blocks = (items + 255) / 256;
+  return (unsigned)(blocks < 16384 ? blocks : 16384);
+}
+
+extern "C" int semipd_add_stream(const void* y, int64_t y_ld, const void* more, int n_more, float* stream, int64_t stream_ld, void* out,
+                                 int64_t out_ld, int64_t rows, int64_t width, int dtype, void* stream_handle) {
+  SEMIPD_CHECK_ARG(rows >= 0 && width > 0 && n_more >= 0, SEMIPD_EINVAL, "add_stream: bad sizes");
+  if (rows == 0) return 0;
+  SEMIPD_CHECK_ARG(stream && (y || n_more > 0 || out) && (n_more == 0 || more), SEMIPD_EINVAL, "add_stream: null pointer");
+  const int64_t esz = dtype == SEMIPD_F32 ? 4 : 2;
+  const bool vec = width % 8 == 0 && aligned16(y) && (y_ld * esz) % 16 == 0 && aligned16(more) && aligned16(stream) && stream_ld % 4 == 0 &&
+                   aligned16(out) && (out_ld * esz) % 16 == 0;
+  SEMIPD_DISPATCH_DTYPE(dtype, T, {
+    if (vec)
+      hipLaunchKernelGGL((add_stream_kernel<T, 8>), dim3(grid_for(rows * (width / 8))), dim3(256), 0, as_stream(stream_handle), (const T*)y,
+                         y_ld, (const T*)more, n_more, stream, stream_ld, (T*)out, out_ld, rows, width);
+    else
+      hipLaunchKernelGGL((add_stream_kernel<T, 1>), dim3(grid_for(rows * width)), dim3(256), 0, as_stream(stream_handle), (const T*)y, y_ld,
+                         (const T*)more, n_more, stream, stream_ld, (T*)out, out_ld, rows, width);
+  });
+  return launch_status("add_stream");
+}
+
+extern "C" int semipd_gelu_mul_rows(const void* z, int64_t z_ld, const int64_t* ids, const void* table, int64_t table_ld, int64_t col,
+                                    void* out, int64_t out_ld, int64_t rows, int64_t width, int dtype, void* stream) {
+  SEMIPD_CHECK_ARG(rows >= 0 && width > 0 && col >= 0 && z_ld >= width && out_ld >= width && table_ld >= col + width, SEMIPD_EINVAL,
+                   "gelu_mul_rows: bad sizes");
+  if (rows == 0) return 0;
+  SEMIPD_CHECK_ARG(z && ids && table && out, SEMIPD_EINVAL, "gelu_mul_rows: null pointer");
+  SEMIPD_DISPATCH_DTYPE(dtype, T,
+                        hipLaunchKernelGGL((gelu_mul_rows_kernel<T>), dim3(grid_for(rows * width)), dim3(256), 0, as_stream(stream),
+                                           (const T*)z, z_ld, ids, (const T*)table, table_ld, col, (T*)out, out_ld, rows, width));
+  return launch_status("gelu_mul_rows");
+}
+
+extern "C" int semipd_glu(const void* x, int64_t x_ld, void* out, int64_t out_ld, int64_t rows, int64_t ff, int64_t up_off, int groups,
+                          const float* topk_weights, const int32_t* topk_ids, int topk, int act, int dtype, void* stream) {
+  SEMIPD_CHECK_ARG(rows >= 0 && ff > 0 && groups > 0 && up_off >= ff && x_ld >= (groups - 1) * 2 * ff + up_off + ff && out_ld >= groups * ff,
+                   SEMIPD_EINVAL, "glu: bad sizes");
+  SEMIPD_CHECK_ARG(act == kGluRelu || act == kGluSilu, SEMIPD_EINVAL, "glu: unknown activation %d", act);
+  if (rows == 0) return 0;
+  SEMIPD_CHECK_ARG(x && out && (topk_weights == nullptr) == (topk_ids == nullptr) && (!topk_ids || topk > 0), SEMIPD_EINVAL,
+                   "glu: null pointer, or routing weights without ids");
+  const int64_t esz = dtype == SEMIPD_F32 ? 4 : 2;
+  const bool vec = ff % 8 == 0 && up_off % 8 == 0 && aligned16(x) && (x_ld * esz) % 16 == 0 && aligned16(out) && (out_ld * esz) % 16 == 0;
+  SEMIPD_DISPATCH_DTYPE(dtype, T, {
+    if (vec)
+      hipLaunchKernelGGL((glu_kernel<T, 8>), dim3(grid_for(rows * groups * (ff / 8))), dim3(256), 0, as_stream(stream), (const T*)x, x_ld,
+                         (T*)out, out_ld, rows, ff, up_off, groups, topk_weights, topk_ids, topk, act);
+    else
+      hipLaunchKernelGGL((glu_kernel<T, 1>), dim3(grid_for(rows * groups * ff)), dim3(256), 0, as_stream(stream), (const T*)x, x_ld,
+                         (T*)out, out_ld, rows, ff, up_off, groups, topk_weights, topk_ids, topk, act);
+  });
+  return launch_status("glu");
 }
 
 extern "C" int semipd_postnorm_stream(const void* y, int64_t y_ld, const void* layer_scale, float* stream, int64_t stream_ld,

@@ -188,7 +188,7 @@ _SIGNATURES = {
     "semipd_state_space": [_vp, _i64, _i64, _i64, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _f32, _vp, _i64, _vp, _i64, _vp, _i64,
                            _vp, _vp, _vp, _vp, _i64, _i64, _i32, _i32, _i32, _i32, _i32, _vp, _i64, _i32, _i32, _vp],
     "semipd_outnorm_stream": [_vp, _i64, _vp, _i64, _vp, _f32, _f32, _vp, _f32, _f32, _vp, _i64, _i64, _i64, _i32, _vp],
-    "semipd_angle_table": [_vp, _vp, _i32, _i64, _vp, _vp],
+    "semipd_angle_table": [_vp, _vp, _i32, _i64, _f32, _vp, _vp],
     "semipd_head_norm_rope_kv_store": [_vp, _i64, _i64, _i32, _i32, _i32, _i32, _i64, _i64, _vp, _vp, _f32, _vp, _i32, _vp, _vp, _vp,
                                        _vp, _vp, _i32, _vp, _vp, _i64, _i32, _i32, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _i32, _vp],
     "semipd_block_means": [_vp, _vp, _i32, _i32, _i32, _i32, _vp, _vp, _i64, _i32, _i32, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _i64, _i32,
@@ -200,10 +200,16 @@ _SIGNATURES = {
     "semipd_matrix_memory_state_width": [_i32, _i32, _i32],
     "semipd_matrix_memory": [_vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _vp, _f32, _vp, _f32, _vp, _i64, _vp, _i64, _vp,
                              _vp, _vp, _vp, _i64, _i64, _i32, _i32, _i32, _f32, _vp, _i64, _i32, _i32, _vp],
+    "semipd_add_stream": [_vp, _i64, _vp, _i32, _vp, _i64, _vp, _i64, _i64, _i64, _i32, _vp],
+    "semipd_gelu_mul_rows": [_vp, _i64, _vp, _vp, _i64, _i64, _vp, _i64, _i64, _i64, _i32, _vp],
+    "semipd_glu": [_vp, _i64, _vp, _i64, _i64, _i64, _i64, _i32, _vp, _vp, _i32, _i32, _i32, _vp],
+    "semipd_linear_attention_workspace": [_i64, _i64, _i32, _i32, _i32, _i32, _i32],
+    "semipd_linear_attention": [_vp, _i64, _i64, _i64, _i64, _i64, _i64, _i32, _vp, _vp, _f32, _vp, _i32, _vp, _i32, _f32, _i32, _vp,
+                                _i64, _vp, _i64, _vp, _vp, _vp, _vp, _i64, _i64, _i32, _i32, _i32, _f32, _vp, _i64, _i32, _i32, _vp],
 }
 _RESTYPES = {"semipd_last_error": C.c_char_p, "semipd_lm_head_argmax_workspace": _sz,
              "semipd_linear_workspace": _sz, "semipd_stream_linear_workspace": _sz, "semipd_dense_gemm_report": _sz, "semipd_ar_meta_size": _sz, "semipd_ar_region_size": _sz,
-             "semipd_matrix_memory_workspace": _i64, "semipd_matrix_memory_state_width": _i64,
+             "semipd_matrix_memory_workspace": _i64, "semipd_linear_attention_workspace": _i64, "semipd_matrix_memory_state_width": _i64,
              "semipd_min_gru_workspace": _i64, "semipd_delta_rule_work_width": _i64, "semipd_state_space_work_width": _i64}
 
 EXPORTED_SYMBOLS = tuple(_SIGNATURES)
@@ -221,6 +227,7 @@ MODEL_SOURCES = {
     "Penozen": ("local_attention.hip", "layernorm.hip", "delta_rule.hip"),
     "Tibenex": ("local_attention.hip", "layernorm.hip", "state_space.hip"),
     "Gukidra": ("local_attention.hip", "attention_prep.hip", "layernorm.hip", "matrix_memory.hip"),
+    "Tebalorn": ("local_attention.hip", "attention_prep.hip", "layernorm.hip", "linear_attention.hip"),
 }
 
 

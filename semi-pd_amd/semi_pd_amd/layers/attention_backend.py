@@ -250,14 +250,15 @@ class HipAttnBackend(AttentionBackend):
 
 
     # ---- block-local attention with a sink term: prompt portions and decode steps over the pools -------------------
-    def forward_local(self, q, layer, forward_batch: ForwardBatch, gate=None, sink=None):
+    def forward_local(self, q, layer, forward_batch: ForwardBatch, gate=None, sink=None, out=None):
         """Attention for layers whose keys and values are in the pool already (the model stored them with the step that
         prepares q): q [T, heads * head_dim] (may be a column range), keys found through req_to_token, so an extend batch
         -- whole prompts, portions with a cached prefix, single tokens of running requests side by side -- and a decode
         batch are the same call.  Mask and cap come from the layer descriptor; `sink` (fp32 [heads], the module's parameter) adds
-        exp(sink) to each head's softmax denominator; `gate` multiplies sigmoid(gate) in."""
+        exp(sink) to each head's softmax denominator; `gate` multiplies sigmoid(gate) in; `out` may be a column range of a wider
+        buffer (the input of an output projection that others write next to)."""
         T = q.shape[0]
-        o = torch.empty((T, layer.tp_q_head_num * layer.v_head_dim), dtype=q.dtype, device=q.device)
+        o = out if out is not None else torch.empty((T, layer.tp_q_head_num * layer.v_head_dim), dtype=q.dtype, device=q.device)
         pool = forward_batch.token_to_kv_pool
         if forward_batch.forward_mode.is_decode():
             q_start = q_len = None

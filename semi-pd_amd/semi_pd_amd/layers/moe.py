@@ -85,9 +85,13 @@ def _local_ids(topk_ids: torch.Tensor, expert_offset: int) -> torch.Tensor:
     return topk_ids if expert_offset == 0 else (topk_ids - expert_offset).to(torch.int32)
 
 
-def _finish(c3: torch.Tensor, out_scale: float, out_addend: Optional[torch.Tensor]) -> torch.Tensor:
+def _finish(c3: torch.Tensor, out_scale: float, out_addend: Optional[torch.Tensor], sum_rows: bool = True) -> torch.Tensor:
     """The sum over the top-k rows; with a scale and / or an addend (DeepseekV2MoE's `* routed_scaling_factor` and
     `+ shared_output`) continued in the same launch with the roundings of the separate ones."""
+    if not sum_rows:
+        if out_scale != 1.0 or out_addend is not None:
+            raise RuntimeError("fused_experts: a scale or an addend belongs to the sum")
+        return c3
     if out_scale == 1.0 and out_addend is None:
         return ops.moe_sum(c3)
     return ops.moe_sum_scale_add(c3, out_scale, out_addend)
@@ -95,13 +99,16 @@ def _finish(c3: torch.Tensor, out_scale: float, out_addend: Optional[torch.Tenso
 
 def fused_experts(hidden_states: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor, topk_weights: torch.Tensor,
                   topk_ids: torch.Tensor, expert_offset: int = 0, partial_experts: bool = False,
-                  out_scale: float = 1.0, out_addend: Optional[torch.Tensor] = None) -> torch.Tensor:
+                  out_scale: float = 1.0, out_addend: Optional[torch.Tensor] = None, sum_rows: bool = True) -> torch.Tensor:
     """fused_experts_impl (fused_moe.py:961-1165), bf16/f16 path.  hidden [T, K]; w1 [E, 2N, K];
-    w2 [E, K, N]; returns [T, K].  partial_experts: w1 / w2 hold only the experts [expert_offset, expert_offset + E)."""
+    w2 [E, K, N]; returns [T, K].  partial_experts: w1 / w2 hold only the experts [expert_offset, expert_offset + E).
+    sum_rows=False: the weighted rows of a token's experts [T, k, K], for a consumer that sums them itself."""
     topk_ids = _local_ids(topk_ids, expert_offset)
     T, K = hidden_states.shape
     E, N2, _ = w1.shape
     if T == 0:   # an empty batch (an idle DP / EP rank): nothing to route, and no block size to divide by
+        if not sum_rows:
+            return hidden_states.new_zeros((0, topk_ids.shape[1], K))
         return out_addend if out_addend is not None else hidden_states.new_zeros((0, K))
     topk = topk_ids.shape[1]
     dev, dt = hidden_states.device, hidden_states.dtype
@@ -138,7 +145,7 @@ def fused_experts(hidden_states: torch.Tensor, w1: torch.Tensor, w2: torch.Tenso
         ops.moe_stream_gemm(hidden_states, w1, c2, None, sorted_ids, expert_ids, num_post_pad, numel, topk, False, block_m, True)
         c3 = (torch.zeros if partial_experts else torch.empty)((numel, K), dtype=dt, device=dev)
         ops.moe_stream_gemm(c2, w2, c3, topk_weights.reshape(-1), sorted_ids, expert_ids, num_post_pad, numel, 1, True, block_m)
-        return _finish(c3.view(T, topk, K), out_scale, out_addend)
+        return _finish(c3.view(T, topk, K), out_scale, out_addend, sum_rows)
     if tall:
         c2 = torch.empty((numel, N2 // 2), dtype=dt, device=dev)
         ops.moe_gemm_tall(hidden_states, w1, c2, None, sorted_ids, expert_ids, num_post_pad, numel, topk, False, True,
@@ -146,7 +153,7 @@ def fused_experts(hidden_states: torch.Tensor, w1: torch.Tensor, w2: torch.Tenso
         c3 = (torch.zeros if partial_experts else torch.empty)((numel, K), dtype=dt, device=dev)
         ops.moe_gemm_tall(c2, w2, c3, topk_weights.reshape(-1), sorted_ids, expert_ids, num_post_pad, numel, 1, True, False,
                           block_m=block_m)
-        return _finish(c3.view(T, topk, K), out_scale, out_addend)
+        return _finish(c3.view(T, topk, K), out_scale, out_addend, sum_rows)
     # prefill-sized calls: SiLU * mul in GEMM1's epilogue (no [T * k, 2N] intermediate); same bits as the two calls
     c2 = ops.moe_grouped_gemm_silu(hidden_states, w1, sorted_ids, expert_ids, num_post_pad, numel, topk, block_m)
     if c2 is None:
@@ -157,7 +164,7 @@ def fused_experts(hidden_states: torch.Tensor, w1: torch.Tensor, w2: torch.Tenso
     c3 = (torch.zeros if partial_experts else torch.empty)((numel, K), dtype=dt, device=dev)
     ops.moe_grouped_gemm(c2, w2, c3, topk_weights.reshape(-1), sorted_ids, expert_ids, num_post_pad, numel, 1, True,
                          block_m)
-    return _finish(c3.view(T, topk, K), out_scale, out_addend)
+    return _finish(c3.view(T, topk, K), out_scale, out_addend, sum_rows)
 
 
 def fused_experts_fp8(hidden_states: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor, w1_scale: torch.Tensor,
@@ -554,3 +561,49 @@ class ClampedGatedMoE(nn.Module):
             y = ops.clamped_glu(u, self.limit, self.alpha, groups=E, topk_weights=topk_weights, topk_ids=topk_ids)
             return dense_linear(y, self.w_down_cat)
         return fused_experts_clamped(hidden_states, self.w13, self.w_down, topk_weights, topk_ids, self.limit, self.alpha)
+
+
+# ---- gated experts whose weights are the softmax over the chosen logits ------------------------------------------------------
+class GatedMoE(nn.Module):
+    """Mixture of silu-gated feed-forward experts, down(silu(gate x) * up x): the top_k largest router logits are chosen, their
+    softmax weighs the experts.  One GPU per replica.  The router weight is kept in fp32 and multiplied in fp32 (its input is the
+    activation-type rows).  `expert_rows` leaves the sum over a token's experts to whoever adds them to the residual stream.
+    fp32 models and widths the grouped kernels refuse evaluate every expert on every token through two plain GEMMs."""
+
+    def __init__(self, num_experts: int, top_k: int, hidden_size: int, intermediate_size: int, params_dtype=None):
+        super().__init__()
+        if not 0 < top_k <= num_experts:
+            raise ValueError(f"GatedMoE: top {top_k} of {num_experts} experts")
+        self.num_experts, self.top_k = num_experts, top_k
+        self.router = nn.Parameter(torch.empty(num_experts, hidden_size, dtype=torch.float32), requires_grad=False)
+        self.w13 = nn.Parameter(torch.empty(num_experts, 2 * intermediate_size, hidden_size, dtype=params_dtype), requires_grad=False)
+        self.w_down = nn.Parameter(torch.empty(num_experts, hidden_size, intermediate_size, dtype=params_dtype), requires_grad=False)
+        self.w_down_cat: Optional[torch.Tensor] = None
+
+    def side_by_side(self) -> bool:
+        return (self.w13.dtype == torch.float32 or self.w13.shape[2] % 8 != 0 or self.w_down.shape[2] % 8 != 0
+                or os.environ.get("SEMIPD_MOE_SIDE_BY_SIDE") == "1")
+
+    def post_load_weights(self):
+        if self.side_by_side():
+            E, K, F = self.w_down.shape
+            self.w_down_cat = self.w_down.permute(1, 0, 2).reshape(K, E * F).contiguous()
+
+    def route(self, hidden_states: torch.Tensor):
+        # (the softmax over all logits, the chosen ones divided by their sum: the softmax over the chosen logits)
+        return ops.topk_softmax(ops.router_logits(hidden_states, self.router), self.top_k, True)
+
+    def expert_rows(self, hidden_states: torch.Tensor) -> torch.Tensor:
+        """[T, n, W]: rows whose sum over n is the mixture's output (n = top_k; 1 where the experts go side by side)."""
+        topk_weights, topk_ids = self.route(hidden_states)
+        if self.w_down_cat is not None:
+            from semi_pd_amd.layers.basic import dense_linear
+            E, F2, K = self.w13.shape
+            u = dense_linear(hidden_states, self.w13.view(E * F2, K))
+            y = ops.glu(u, F2 // 2, "silu", groups=E, topk_weights=topk_weights, topk_ids=topk_ids)
+            return dense_linear(y, self.w_down_cat).unsqueeze(1)
+        return fused_experts(hidden_states, self.w13, self.w_down, topk_weights, topk_ids, sum_rows=False)
+
+    def forward(self, hidden_states: torch.Tensor) -> torch.Tensor:
+        rows = self.expert_rows(hidden_states)
+        return rows[:, 0] if rows.shape[1] == 1 else ops.moe_sum(rows)

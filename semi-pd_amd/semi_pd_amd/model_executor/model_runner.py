@@ -60,6 +60,9 @@ def build_model(model_config, dtype):
     if arch == "Gukidra":
         from semi_pd_amd.models.gukidra import GukidraForCausalLM
         return GukidraForCausalLM(model_config, dtype)
+    if arch == "Tebalorn":
+        from semi_pd_amd.models.tebalorn import TebalornForCausalLM
+        return TebalornForCausalLM(model_config, dtype)
     raise ValueError(f"unsupported architecture {arch}")
 
 

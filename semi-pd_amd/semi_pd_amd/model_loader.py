@@ -29,9 +29,10 @@ def _config_classes():
     from semi_pd_amd.models.kudirax import KudiraxConfig
     from semi_pd_amd.models.opt import OPTConfig
     from semi_pd_amd.models.penozen import PenozenConfig
+    from semi_pd_amd.models.tebalorn import TebalornConfig
     from semi_pd_amd.models.tibenex import TibenexConfig
     from semi_pd_amd.models.tigotar import TigotarConfig
-    return {"Gukidra": GukidraConfig, "Tibenex": TibenexConfig, "Tigotar": TigotarConfig, "Penozen": PenozenConfig, "LlamaForCausalLM": LlamaConfig, "OPTForCausalLM": OPTConfig,
+    return {"Tebalorn": TebalornConfig, "Gukidra": GukidraConfig, "Tibenex": TibenexConfig, "Tigotar": TigotarConfig, "Penozen": PenozenConfig, "LlamaForCausalLM": LlamaConfig, "OPTForCausalLM": OPTConfig,
             "DeepseekV2ForCausalLM": DeepseekV2Config, "DeepseekV3ForCausalLM": DeepseekV2Config,
             "Kudirax": KudiraxConfig}
 
@@ -67,7 +68,10 @@ def config_from_hf_dict(d: dict):
 
 def load_hf_config(model_path: str):
     with open(os.path.join(model_path, "config.json")) as f:
-        return config_from_hf_dict(json.load(f))
+        cfg = config_from_hf_dict(json.load(f))
+    if hasattr(cfg, "read_tensor_shapes"):       # designs with sizes that only the checkpoint's tensors give
+        cfg.read_tensor_shapes(safetensors_shapes(model_path))
+    return cfg
 
 
 # ----------------------------------------------------------------------------------- weights
@@ -87,6 +91,17 @@ def safetensors_weights_iterator(model_path: str) -> Iterator[Tuple[str, torch.T
         with safe_open(fpath, framework="pt", device="cpu") as f:
             for k in f.keys():
                 yield k, f.get_tensor(k)
+
+
+def safetensors_shapes(model_path: str) -> Dict[str, Tuple[int, ...]]:
+    """Shape of every tensor of every *.safetensors shard, from the files' headers (no shards: empty)."""
+    from safetensors import safe_open
+    shapes = {}
+    for fpath in sorted(glob.glob(os.path.join(model_path, "*.safetensors"))):
+        with safe_open(fpath, framework="pt", device="cpu") as f:
+            for k in f.keys():
+                shapes[k] = tuple(f.get_slice(k).get_shape())
+    return shapes
 
 
 class _Stacker:
@@ -413,6 +428,75 @@ def _gukidra_items(config, weights):
         raise RuntimeError(f"checkpoint ended with incomplete stacked parameters: {list(st.pending)[:4]}")
 
 
+_TEBALORN_RE = re.compile(r"^l(\d+)\.(mix|mlp|norm1|side)(?:\.(.+))?$")
+_TEBALORN_LEAF = {"attention": {"sink": "sink"}, "gla": {"norm": "out_norm", "a2": "a2", "a2.b": "a2_bias"}, "lightning": {"norm": "out_norm"}}
+_TEBALORN_SIDE = {"gate": "gate", "proj": "proj", "norm": "norm.weight"}
+
+
+def _tebalorn_items(config, weights):
+    """Tebalorn checkpoint names (embed, side.embed, l<i>.norm1, l<i>.mix.q|k|v|o plus sink of an attention layer, g|norm of a linear
+    attention, a1|a2|a2.b of a decay per channel, l<i>.mlp.gate|up|down of a dense feed-forward, l<i>.mlp.router|e<j>.*|shared.* of a
+    mixture, l<i>.side.gate|proj|norm, final.norm, head) -> product parameters: the mixer's parts and gate | up (dense or shared)
+    stack into the layer's input projection, each brought to a multiple of 8 rows with zeros; o and down side by side into its
+    output projection; every expert's gate and up rows into [E, 2F, W]."""
+    from semi_pd_amd.models.tebalorn import mixer_parts
+    st = _Stacker()
+    top = {"embed": "embed.weight", "side.embed": "side_table", "head": "head.weight", "final.norm": "final_norm.weight"}
+
+    def unknown(name):
+        return KeyError(f"checkpoint tensor {name} has no counterpart in a Tebalorn model")
+
+    for name, t in weights:
+        if name in top:
+            yield top[name], t
+            continue
+        m = _TEBALORN_RE.match(name)
+        if not m or int(m.group(1)) >= len(config.layers):
+            raise unknown(name)
+        i, part, leaf = int(m.group(1)), m.group(2), m.group(3)
+        base, lc = f"layers.{i}.", config.layers[i]
+        ins = [p for p, _ in mixer_parts(lc)]
+        n_in, n_out = len(ins) + (2 if lc.ff else 0), 2 if lc.ff else 1
+        if part == "norm1":
+            if leaf is not None:
+                raise unknown(name)
+            yield base + "norm1.weight", t
+        elif part == "side":
+            if leaf not in _TEBALORN_SIDE:
+                raise unknown(name)
+            yield base + "side." + _TEBALORN_SIDE[leaf], t
+        else:
+            index = None
+            if part == "mix" and leaf in ins:
+                index = ins.index(leaf)
+            elif part == "mlp" and lc.ff and leaf in (("shared.gate", "shared.up") if lc.experts else ("gate", "up")):
+                index = len(ins) + int(leaf.endswith("up"))
+            if index is not None:
+                pad = -t.shape[0] % 8
+                yield from st.add(base + "in_proj.weight", index, n_in, torch.cat([t, t.new_zeros(pad, t.shape[1])], 0) if pad else t)
+            elif part == "mix" and leaf == "o":
+                yield from st.add(base + "out_proj.weight", 0, n_out, t, dim=1)
+            elif part == "mlp" and lc.ff and leaf == ("shared.down" if lc.experts else "down"):
+                yield from st.add(base + "out_proj.weight", 1, n_out, t, dim=1)
+            elif part == "mix" and leaf in _TEBALORN_LEAF[lc.kind]:
+                yield base + "mix." + _TEBALORN_LEAF[lc.kind][leaf], t
+            elif part == "mlp" and lc.experts and leaf == "router":
+                yield base + "moe.router", t
+            else:
+                em = re.match(r"^e(\d+)\.(gate|up|down)$", leaf or "") if part == "mlp" else None
+                if not em or int(em.group(1)) >= lc.experts:
+                    raise unknown(name)
+                e, which = int(em.group(1)), em.group(2)
+                if which == "down":
+                    yield from st.add(base + "moe.w_down", e, lc.experts, t, dim=None)
+                else:
+                    # (gate rows of expert e, then its up rows; the experts' blocks follow each other)
+                    for done_name, full in st.add(base + "moe.w13", 2 * e + (which == "up"), 2 * lc.experts, t):
+                        yield done_name, full.reshape(lc.experts, 2 * lc.expert_ff, full.shape[1])
+    if st.pending:
+        raise RuntimeError(f"checkpoint ended with incomplete stacked parameters: {list(st.pending)[:4]}")
+
+
 _EXPERT_RE = re.compile(r"^(.*\.mlp\.experts)\.(\d+)\.(gate_proj|up_proj|down_proj)\.(weight|weight_scale_inv)$")
 
 
@@ -430,6 +514,9 @@ def product_items(config, weights: Iterable[Tuple[str, torch.Tensor]]) -> Iterat
         return
     if arch == "Tibenex":
         yield from _tibenex_items(config, weights)
+        return
+    if arch == "Tebalorn":
+        yield from _tebalorn_items(config, weights)
         return
     if arch == "Gukidra":
         yield from _gukidra_items(config, weights)

@@ -2048,13 +2048,13 @@ def outnorm_stream(y: torch.Tensor, stream: torch.Tensor, weight: torch.Tensor, 
     return out
 
 
-def angle_table(positions: torch.Tensor, freq: torch.Tensor) -> torch.Tensor:
-    """fp32 [T, len(freq), 2]: cos and sin of position * freq (csrc/attention_prep.hip)."""
+def angle_table(positions: torch.Tensor, freq: torch.Tensor, factor: float = 1.0) -> torch.Tensor:
+    """fp32 [T, len(freq), 2]: cos and sin of position * freq, times factor (csrc/attention_prep.hip)."""
     if positions.dtype != torch.int64 or not positions.is_contiguous() or freq.dtype != torch.float32 or not freq.is_contiguous():
         raise RuntimeError("angle_table: int64 positions, fp32 frequencies")
     T, half = positions.shape[0], freq.numel()
     out = torch.empty((T, half, 2), dtype=torch.float32, device=positions.device)
-    check(_lib.load().semipd_angle_table(ptr(positions), ptr(freq), half, T, ptr(out), current_stream(positions.device)), "angle_table")
+    check(_lib.load().semipd_angle_table(ptr(positions), ptr(freq), half, T, float(factor), ptr(out), current_stream(positions.device)), "angle_table")
     return out
 
 
@@ -2075,15 +2075,15 @@ def _check_means(name: str, means, k_buffer: torch.Tensor, v_buffer: torch.Tenso
 
 
 def head_norm_rope_kv_store(qkv: torch.Tensor, num_q_heads: int, num_kv_heads: int, qk_dim: int, v_dim: int, k_off: int, v_off: int,
-                            q_weight: torch.Tensor, k_weight: Optional[torch.Tensor], eps: float, qk_angles: Optional[torch.Tensor],
-                            rot_dims: int, v_angles: Optional[torch.Tensor], k_buffer: Optional[torch.Tensor],
+                            q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], eps: float,
+                            qk_angles: Optional[torch.Tensor], rot_dims: int, v_angles: Optional[torch.Tensor], k_buffer: Optional[torch.Tensor],
                             v_buffer: Optional[torch.Tensor], loc: Optional[torch.Tensor], means=None,
                             positions: Optional[torch.Tensor] = None, req_to_token: Optional[torch.Tensor] = None,
                             req_pool_indices: Optional[torch.Tensor] = None, seq_lens: Optional[torch.Tensor] = None,
                             q_start: Optional[torch.Tensor] = None, q_len: Optional[torch.Tensor] = None) -> None:
     """Rows of `qkv` hold q | k | v at columns 0, k_off, v_off (num_kv_heads = 0: queries only).  Every q / k head to unit RMS times
-    a weight [qk_dim], its first rot_dims elements turned in pairs (i, i + rot_dims / 2) by qk_angles; every v head turned in
-    pairs (m, m + v_dim / 2) by v_angles; q in place, k / v into the pools at `loc`.  `means` = (block size, key means, value
+    a weight [qk_dim] (no norm without weights), its first rot_dims elements turned in pairs (i, i + rot_dims / 2) by qk_angles;
+    every v head turned in pairs (m, m + v_dim / 2) by v_angles (None: v passes); q in place, k / v into the pools at `loc`.  `means` = (block size, key means, value
     means): the blocks that the batch completes get their means as well (csrc/attention_prep.hip)."""
     name = "head_norm_rope_kv_store"
     if qkv.dim() != 2 or qkv.stride(1) != 1:
@@ -2096,7 +2096,8 @@ def head_norm_rope_kv_store(qkv: torch.Tensor, num_q_heads: int, num_kv_heads: i
         _check_angles(name, qk_angles, T, rot_dims // 2)
     B = 0
     if num_kv_heads:
-        _check_angles(name, v_angles, T, v_dim // 2)
+        if v_angles is not None:
+            _check_angles(name, v_angles, T, v_dim // 2)
         if loc.dtype != torch.int64 or loc.shape[0] != T:
             raise RuntimeError(f"{name}: one int64 pool slot per row")
         for buf, size in ((k_buffer, qk_dim), (v_buffer, v_dim)):
@@ -2212,4 +2213,126 @@ def matrix_memory(proj: torch.Tensor, offsets, num_heads: int, qk_dim: int, v_di
                                    ptr(state_indices), ptr(seq_lens), ptr(q_start), ptr(q_len), B, T, num_heads, qk_dim, v_dim,
                                    float(qk_dim) ** -0.5, ptr(out), out.stride(0), int(form), dtype_code(proj.dtype),
                                    current_stream(proj.device)), "matrix_memory")
+    return out
+
+
+# ---- two sublayers on one input, a per-token table beside the stream, gated activations over column ranges, linear attention -------
+def add_stream(y: Optional[torch.Tensor], stream: torch.Tensor, more: Optional[torch.Tensor] = None, dtype=None) -> torch.Tensor:
+    """stream (fp32 [rows, width], in place) += y + more.sum(1) (y [rows, width], more [rows, n, width] contiguous, one type);
+    returns the new stream in that type (csrc/layernorm.hip: semipd_add_stream)."""
+    if stream.dim() != 2 or stream.dtype != torch.float32 or stream.stride(1) != 1:
+        raise RuntimeError("add_stream: the stream is fp32 [rows, width] with contiguous rows")
+    rows, width = stream.shape
+    dt = y.dtype if y is not None else (more.dtype if more is not None else dtype)
+    if y is not None and (y.shape != stream.shape or y.stride(1) != 1):
+        raise RuntimeError("add_stream: y is shaped like the stream, with contiguous rows")
+    if more is not None and (more.dim() != 3 or more.shape[0] != rows or more.shape[2] != width or not more.is_contiguous() or more.dtype != dt):
+        raise RuntimeError("add_stream: more is contiguous [rows, n, width] of y's type")
+    out = torch.empty((rows, width), dtype=dt, device=stream.device)
+    check(_lib.load().semipd_add_stream(ptr(y), y.stride(0) if y is not None else 0, ptr(more), more.shape[1] if more is not None else 0,
+                                        ptr(stream), stream.stride(0), ptr(out), out.stride(0), rows, width, dtype_code(dt),
+                                        current_stream(stream.device)), "add_stream")
+    return out
+
+
+def gelu_mul_rows(z: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, col: int) -> torch.Tensor:
+    """gelu_tanh(z [T, P]) * table[ids, col: col + P] (csrc/layernorm.hip: semipd_gelu_mul_rows)."""
+    T, P = z.shape
+    if z.stride(1) != 1 or ids.dtype != torch.int64 or ids.shape != (T,) or not ids.is_contiguous() or table.dim() != 2 \
+            or table.stride(1) != 1 or table.dtype != z.dtype or not 0 <= col <= table.shape[1] - P:
+        raise RuntimeError("gelu_mul_rows: z [T, P], int64 ids [T], table [V, >= col + P] of z's type")
+    out = torch.empty((T, P), dtype=z.dtype, device=z.device)
+    check(_lib.load().semipd_gelu_mul_rows(ptr(z), z.stride(0), ptr(ids), ptr(table), table.stride(0), int(col), ptr(out), out.stride(0),
+                                           T, P, dtype_code(z.dtype), current_stream(z.device)), "gelu_mul_rows")
+    return out
+
+
+GLU_ACTIVATIONS = {"relu": 0, "silu": 1}
+
+
+def glu(x: torch.Tensor, ff: int, act: str, out: Optional[torch.Tensor] = None, up_off: Optional[int] = None, groups: int = 1,
+        topk_weights: Optional[torch.Tensor] = None, topk_ids: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x [rows, groups * 2 * ff] (may be a column range), every group [gate ff | up ff] (up at up_off with one group): act(gate) * up
+    -> [rows, groups * ff], `out` may be a column range; with routing, times the routing weight of the group's expert for the
+    row (0 if the row does not use it) (csrc/layernorm.hip: semipd_glu)."""
+    rows = x.shape[0]
+    up = ff if up_off is None else int(up_off)
+    if x.dim() != 2 or x.stride(1) != 1 or up < ff or (groups > 1 and up != ff) or x.shape[1] < (groups - 1) * 2 * ff + up + ff:
+        raise RuntimeError("glu: x is [rows, groups * 2 * ff] with contiguous rows")
+    k = 0
+    if (topk_weights is None) != (topk_ids is None):
+        raise RuntimeError("glu: routing weights come with their ids")
+    if topk_ids is not None:
+        if topk_weights.dtype != torch.float32 or topk_ids.dtype != torch.int32 or topk_weights.shape != topk_ids.shape \
+                or topk_ids.shape[0] != rows or not topk_weights.is_contiguous() or not topk_ids.is_contiguous():
+            raise RuntimeError("glu: topk_weights fp32 / topk_ids int32 [rows, k] contiguous")
+        k = topk_ids.shape[1]
+    if out is None:
+        out = torch.empty((rows, groups * ff), dtype=x.dtype, device=x.device)
+    if out.shape != (rows, groups * ff) or out.dtype != x.dtype or out.stride(1) != 1:
+        raise RuntimeError("glu: out is [rows, groups * ff] of x's type with contiguous rows")
+    check(_lib.load().semipd_glu(ptr(x), x.stride(0), ptr(out), out.stride(0), rows, ff, up, groups, ptr(topk_weights), ptr(topk_ids), k,
+                                 GLU_ACTIVATIONS[act], dtype_code(x.dtype), current_stream(x.device)), "glu")
+    return out
+
+
+DECAY_POWERS = 65            # powers 0 .. 64 of a head's decay: what a chunk of 64 tokens needs
+
+
+def decay_powers(decay) -> torch.Tensor:
+    """fp32 [H, 65]: the powers of each head's decay, the decay itself rounded to fp32 first (as the token-by-token form uses it)."""
+    d = torch.tensor([float(x) for x in decay], dtype=torch.float32).double()
+    return (d.unsqueeze(1) ** torch.arange(DECAY_POWERS, dtype=torch.float64)).float().contiguous()
+
+
+def linear_attention(proj: torch.Tensor, offsets, num_heads: int, qk_dim: int, v_dim: int, q_scale: float, norm_weight: torch.Tensor,
+                     norm_together: bool, gate: str, eps: float, state: torch.Tensor, state_indices: torch.Tensor,
+                     seq_lens: torch.Tensor, q_start: Optional[torch.Tensor], q_len: Optional[torch.Tensor],
+                     powers: Optional[torch.Tensor] = None, a_off: int = 0, a2: Optional[torch.Tensor] = None,
+                     a2_bias: Optional[torch.Tensor] = None, tau: float = 1.0, qkv_silu: bool = False,
+                     out: Optional[torch.Tensor] = None, form: int = 0) -> torch.Tensor:
+    """Linear attention with decays behind its projection GEMM (csrc/linear_attention.hip).  offsets: columns of q, k, v and the
+    output gate in the rows of `proj`.  Decay: `powers` (decay_powers: one constant per head), or a2 [H * D, rank] / a2_bias fp32
+    [H * D] / tau over the columns a_off .. a_off + rank (one per key channel).  norm_weight [H * E] (all heads together) or [E]
+    (each head); gate "sigmoid" | "silu"; state fp32 [slots, H * D * E] is a column range of the requests' state rows.  Returns
+    [T, H * E] (`out` may be a column range)."""
+    name = "linear_attention"
+    T, B = proj.shape[0], state_indices.shape[0]
+    qk, inner = num_heads * qk_dim, num_heads * v_dim
+    if proj.dim() != 2 or proj.stride(1) != 1:
+        raise RuntimeError(f"{name}: proj is 2-D with contiguous rows")
+    q_off, k_off, v_off, g_off = (int(o) for o in offsets)
+    if min(offsets) < 0 or max(q_off + qk, k_off + qk, v_off + inner, g_off + inner) > proj.shape[1]:
+        raise RuntimeError(f"{name}: a column range leaves the row")
+    if (powers is None) == (a2 is None):
+        raise RuntimeError(f"{name}: a decay per head or one per channel")
+    rank = 0
+    if powers is not None:
+        if powers.dtype != torch.float32 or powers.shape != (num_heads, DECAY_POWERS) or not powers.is_contiguous():
+            raise RuntimeError(f"{name}: powers is fp32 [H, {DECAY_POWERS}] contiguous")
+    else:
+        rank = a2.shape[1]
+        if a2.shape[0] != qk or a2.dtype != proj.dtype or not a2.is_contiguous() or a2_bias.dtype != torch.float32 \
+                or a2_bias.shape != (qk,) or not a2_bias.is_contiguous() or a_off < 0 or a_off + rank > proj.shape[1]:
+            raise RuntimeError(f"{name}: a2 is contiguous [H * D, rank] of the activation type, a2_bias fp32 [H * D]")
+    if norm_weight.shape != ((inner if norm_together else v_dim),) or norm_weight.dtype != proj.dtype or not norm_weight.is_contiguous():
+        raise RuntimeError(f"{name}: norm_weight is contiguous [{'H * E' if norm_together else 'E'}] of the activation type")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] != qk * v_dim or state.stride(1) != 1:
+        raise RuntimeError(f"{name}: state is fp32 [slots, H * D * E]")
+    if state_indices.dtype != torch.int64 or seq_lens.dtype != torch.int64 or seq_lens.shape[0] != B:
+        raise RuntimeError(f"{name}: state_indices / seq_lens are int64 [B]")
+    _batch_rows(name, T, B, q_start, q_len)
+    if out is None:
+        out = torch.empty((T, inner), dtype=proj.dtype, device=proj.device)
+    if out.shape != (T, inner) or out.dtype != proj.dtype or out.stride(1) != 1:
+        raise RuntimeError(f"{name}: out is [T, H * E] of the activation type with contiguous rows")
+    lib = _lib.load()
+    dt = dtype_code(proj.dtype)
+    work = torch.empty(int(lib.semipd_linear_attention_workspace(T, B, num_heads, qk_dim, v_dim, int(q_start is not None), dt)),
+                       dtype=torch.float32, device=proj.device)
+    check(lib.semipd_linear_attention(ptr(proj), proj.stride(0), q_off, k_off, v_off, g_off, int(a_off), rank, ptr(a2), ptr(a2_bias),
+                                      float(tau), ptr(powers), int(qkv_silu), ptr(norm_weight), int(norm_together), float(eps),
+                                      {"sigmoid": 0, "silu": 1}[gate], ptr(work), work.numel(), ptr(state), state.stride(0),
+                                      ptr(state_indices), ptr(seq_lens), ptr(q_start), ptr(q_len), B, T, num_heads, qk_dim, v_dim,
+                                      float(q_scale), ptr(out), out.stride(0), int(form), dt, current_stream(proj.device)), name)
     return out
