@@ -6,7 +6,9 @@ a mixture of experts behind them);
 with `--arch-design tibenex`: Tibenex next to Penozen (fp32 stream, latent attention, a recurrence with a matrix state and a
 short convolution over pooled state rows);
 with `--arch-design gukidra`: Gukidra next to Tibenex (fp32 stream with a norm behind every sublayer, attention and a recurrence
-with a matrix state over pooled state rows, a dense feed-forward), its windowed attention next to Tigotar's window kernel.
+with a matrix state over pooled state rows, a dense feed-forward), its windowed attention next to Tigotar's window kernel;
+with `--arch-design tebalorn`: Tebalorn next to Gukidra (fp32 stream, attention and a recurrence with a matrix state of the same
+size), with its mixture of experts next to Penozen.
 
 Two parts, printed as one JSON object:
   * "models": prefill and decode throughput of a few-layer model of each design at layer sizes of real models, both driven
@@ -924,7 +926,188 @@ def main_gukidra(args) -> dict:
     return result
 
 
+TEBALORN_SIZES = {
+    # name: hidden, ff, vocab, attention heads / kv heads / head size and chunk, linear-attention heads / key size / value size (the
+    # state of a layer as large as that of Gukidra's memory), token-side size, experts (the active sizes sum to ff)
+    "8b-layer": dict(hidden=4096, ff=14336, vocab=32000, heads=32, kv=8, dim=128, chunk=1024, lheads=8, ldim=256, lvdim=512, side=256, experts=8, top=2),
+    "3b-layer": dict(hidden=3072, ff=8192, vocab=32000, heads=24, kv=8, dim=128, chunk=1024, lheads=6, ldim=256, lvdim=512, side=256, experts=8, top=2),
+    "1b-layer": dict(hidden=2048, ff=8192, vocab=32000, heads=32, kv=8, dim=64, chunk=1024, lheads=8, ldim=128, lvdim=256, side=256, experts=16, top=4),
+}
+
+
+def _tebalorn_kernel_pairs(s, gs, dev):
+    """[(what, Tebalorn kernel's record, like kernel's record)]: `s` Tebalorn's layer shape, `gs` Gukidra's at the same size."""
+    from semi_pd_amd import ops
+    from semi_pd_amd.mem_cache.memory_pool import mean_piece
+    dt = torch.bfloat16
+    W, FF, P = s["hidden"], s["ff"], s["side"]
+    out = []
+
+    def rec(tm, nbytes=0.0, flops=0.0, vflops=0.0):
+        frac = max(nbytes / tm / HBM, flops / tm / MFMA, vflops / tm / VALU)
+        return {"us": round(tm * 1e6, 1), "TB_per_s": round(nbytes / tm / 1e12, 2),
+                "TFLOP_per_s": round(max(flops, vflops) / tm / 1e12, 1), "of_roofline": round(frac, 4)}
+
+    B, L = 4, 2048
+    T = B * L
+    B2, C = 32, 2000
+    rows, lens = torch.arange(B, device=dev), torch.full((B,), L, device=dev, dtype=torch.int64)
+    q_start = torch.arange(B, device=dev, dtype=torch.int32) * L
+    q_len = torch.full((B,), L, device=dev, dtype=torch.int32)
+    rows2, lens2 = torch.arange(B2, device=dev), torch.full((B2,), C, device=dev, dtype=torch.int64)
+    st4, st32 = torch.arange(1, B + 1, device=dev), torch.arange(1, B2 + 1, device=dev)
+    r2t = (torch.arange(T, device=dev, dtype=torch.int32) + 1).view(B, L).contiguous()
+    r2t2 = (torch.arange(B2 * C, device=dev, dtype=torch.int32) + 1).view(B2, C).contiguous()
+    # ---- into the stream ---------------------------------------------------------------------------------------------------
+    for Tn in (8192, 32):
+        y = torch.randn(Tn, W, device=dev, dtype=dt)
+        more = torch.randn(Tn, s["top"], W, device=dev, dtype=dt)
+        res = torch.randn(Tn, W, device=dev, dtype=torch.float32)
+        w = torch.zeros(W, device=dev, dtype=dt)
+        t_old = _timed(lambda: ops.outnorm_stream(y, res, w, 1e-5, 1.0))
+        old = rec(t_old, nbytes=Tn * W * (2 + 4 + 4 + 2.0))
+        out.append((f"stream += y, copy, {Tn} rows of {W} (like: stream += norm(y), copy)",
+                    rec(_timed(lambda: ops.add_stream(y, res)), nbytes=Tn * W * (2 + 4 + 4 + 2.0)), old))
+        out.append((f"stream += y + {s['top']} experts' rows, copy, {Tn} rows of {W} (like: stream += norm(y), copy)",
+                    rec(_timed(lambda: ops.add_stream(y, res, more)), nbytes=Tn * W * (2 + 2 * s["top"] + 4 + 4 + 2.0)), old))
+        w1 = torch.ones(W, device=dev, dtype=dt)
+        out.append((f"stream += norm(y), the next layer's norm, {Tn} rows of {W} (like: stream += norm(y), copy)",
+                    rec(_timed(lambda: ops.outnorm_stream(y, res, w, 1e-5, 1.0, next_weight=w1, next_eps=1e-6)), nbytes=Tn * W * (2 + 4 + 4 + 2.0)), old))
+        # gated activation: columns of the merged projection into columns of the output GEMM's input
+        inner = s["lheads"] * s["lvdim"]
+        p = torch.randn(Tn, 4 * inner + 2 * FF, device=dev, dtype=dt)
+        both = torch.empty(Tn, inner + FF, device=dev, dtype=dt)
+        pc = torch.randn(Tn, 2 * FF, device=dev, dtype=dt)
+        out.append((f"relu(gate) * up over column ranges, {Tn} rows of {FF} (like: silu(gate) * up)",
+                    rec(_timed(lambda: ops.glu(p[:, 4 * inner:], FF, "relu", out=both[:, inner:])), nbytes=Tn * FF * 6.0),
+                    rec(_timed(lambda: ops.silu_and_mul(pc)), nbytes=Tn * FF * 6.0)))
+        z = torch.randn(Tn, P, device=dev, dtype=dt)
+        table = torch.randn(s["vocab"], 4 * P, device=dev, dtype=dt)
+        ids = torch.randint(0, s["vocab"], (Tn,), device=dev)
+        pz = torch.randn(Tn, 2 * P, device=dev, dtype=dt)
+        out.append((f"gelu(z) * the token's table row, {Tn} rows of {P} (like: silu(gate) * up)",
+                    rec(_timed(lambda: ops.gelu_mul_rows(z, ids, table, P)), nbytes=Tn * P * 6.0),
+                    rec(_timed(lambda: ops.silu_and_mul(pz)), nbytes=Tn * P * 6.0)))
+        del p, both, pc
+    # ---- attention ---------------------------------------------------------------------------------------------------------
+    H, G, D, N = s["heads"], s["kv"], s["dim"], s["chunk"]
+    E, pool, gN = D, gs["pool"], gs["window"]
+    n_slots = max(T, B2 * C) + 1
+    kp = torch.randn(n_slots, G, D, device=dev, dtype=dt)
+    vp = torch.randn(n_slots, G, E, device=dev, dtype=dt)
+    km = torch.randn(G, n_slots, mean_piece(D, pool), device=dev, dtype=dt)
+    vm = torch.randn(G, n_slots, mean_piece(E, pool), device=dev, dtype=dt)
+    means = (pool, km, vm)
+    nw = torch.ones(D, device=dev, dtype=dt)
+    freq = 10000.0 ** (-2.0 * torch.arange(D // 2, dtype=torch.float32, device=dev) / D)
+    sink = torch.zeros(H, device=dev)
+    for Tn, decode in ((8192, False), (32, True)):
+        p = torch.randn(Tn, (H + G) * D + G * E + H, device=dev, dtype=dt)
+        loc = torch.arange(1, Tn + 1, device=dev) if not decode else r2t2[:, -1].long().contiguous()
+        pos = torch.arange(Tn, device=dev) % L if not decode else torch.full((Tn,), C - 1, device=dev, dtype=torch.int64)
+        tab = ops.angle_table(pos, freq, 1.2)
+        nbytes = Tn * 2.0 * (2 * H * D + 2 * G * (D + E))
+        out.append((f"rotation of q and k + KV store, {Tn} {'decode rows' if decode else 'tokens'}, {H} / {G} heads of {D} / {E} (like: head norms + "
+                    f"rotation of q, k and v + KV store)",
+                    rec(_timed(lambda: ops.head_norm_rope_kv_store(p, H, G, D, E, H * D, (H + G) * D, None, None, 0.0, tab, D, None, kp, vp, loc)), nbytes=nbytes),
+                    rec(_timed(lambda: ops.head_norm_rope_kv_store(p, H, G, D, E, H * D, (H + G) * D, nw, nw, 1e-5, tab, D, tab, kp, vp, loc)), nbytes=nbytes)))
+    q = torch.randn(T, H * D, device=dev, dtype=dt)
+    o = torch.empty(T, H * E, device=dev, dtype=dt)
+    gate = torch.randn(T, H, device=dev, dtype=dt)
+    tab = ops.angle_table(torch.arange(T, device=dev) % L, freq)
+    pairs = B * sum(i % N + 1 for i in range(L))
+    gpairs = B * sum(min(i + 1, gN) + max(0, i - gN + 1) // pool for i in range(L))
+    t_new = _timed(lambda: ops.local_attention_fwd(q, o, kp, vp, r2t, rows, lens, q_start, q_len, L, D ** -0.5, 0.0, N, sink, None))
+    t_old = _timed(lambda: ops.pooled_window_attention_fwd(q, o, kp, vp, means, r2t, rows, lens, q_start, q_len, L, D ** -0.5, gN, sink=sink,
+                                                           gate=gate, turn=tab))
+    out.append((f"prompt attention, {B} x {L} tokens, {H} / {G} heads of {D} / {E}, chunks of {N}, a sink (like: window {gN} + block means of {pool}, turned "
+                f"back, gated)", rec(t_new, flops=2.0 * H * (D + E) * pairs), rec(t_old, flops=2.0 * H * (D + E) * gpairs)))
+    q2 = torch.randn(B2, H * D, device=dev, dtype=dt)
+    o2 = torch.empty(B2, H * E, device=dev, dtype=dt)
+    gate2 = torch.randn(B2, H, device=dev, dtype=dt)
+    tab2 = ops.angle_table(torch.full((B2,), C - 1, device=dev, dtype=torch.int64), freq)
+    nb, seen = max(0, C - gN) // pool, (C - 1) % N + 1
+    splits = max(1, min(16, 256 // (B2 * G * ((H // G + 15) // 16)), (gN + nb) // 128))
+    t_new = _timed(lambda: ops.local_attention_fwd(q2, o2, kp, vp, r2t2, rows2, lens2, None, None, 1, D ** -0.5, 0.0, N, sink, None))
+    t_old = _timed(lambda: ops.pooled_window_attention_fwd(q2, o2, kp, vp, means, r2t2, rows2, lens2, None, None, 1, D ** -0.5, gN, sink=sink,
+                                                           gate=gate2, turn=tab2, n_splits=splits))
+    out.append((f"decode attention, {B2} requests at {C} tokens, {H} / {G} heads of {D} / {E}, chunks of {N} (like: window + block means)",
+                rec(t_new, nbytes=B2 * G * (D + E) * 2.0 * seen), rec(t_old, nbytes=B2 * G * (D + E) * 2.0 * (gN + nb))))
+    # ---- the recurrences ---------------------------------------------------------------------------------------------------
+    MH, MD, ME = gs["mheads"], gs["mdim"], gs["mvdim"]
+    sizes = [MH * MD, MH * MD, MH * ME, MH * ME, MH, MH]
+    offs = [sum(sizes[:i]) for i in range(6)]
+    width = sum(sizes) + -sum(sizes) % 8
+    ib, fb = torch.zeros(MH, device=dev), torch.zeros(MH, device=dev) + 4.0
+    mnw = torch.ones(MH * ME, device=dev, dtype=dt)
+    SW = ops.matrix_memory_state_width(MH, MD, ME)
+    mS = torch.zeros(B2 + 1, -(-SW // 4) * 4, device=dev)[:, :SW]
+    LH, LD, LE, rank = s["lheads"], s["ldim"], s["lvdim"], 16
+    lsizes = [LH * LD, LH * LD, LH * LE, LH * LE, rank]
+    loffs = [sum(lsizes[:i]) for i in range(5)]
+    lS = torch.zeros(B2 + 1, LH * LD * LE, device=dev)
+    a2, ab = torch.randn(LH * LD, rank, device=dev, dtype=dt) * 0.25, torch.zeros(LH * LD, device=dev) + 2.0
+    powers = ops.decay_powers([1.0 - 2.0 ** (-3 - i) for i in range(LH)]).to(dev)
+    nw1, nwa = torch.ones(LE, device=dev, dtype=dt), torch.ones(LH * LE, device=dev, dtype=dt)
+    for Tn, decode in ((T, False), (B2, True)):
+        mp = torch.randn(Tn, width, device=dev, dtype=dt)
+        lp = torch.randn(Tn, sum(lsizes), device=dev, dtype=dt)
+        where = (st32, lens2, None, None) if decode else (st4, lens, q_start, q_len)
+        t_old = _timed(lambda: ops.matrix_memory(mp, offs, MH, MD, ME, ib, fb, 15.0, mnw, 1e-5, mS, *where), iters=10, warm=2)
+        t_g = _timed(lambda: ops.linear_attention(lp, loffs[:4], LH, LD, LE, LD ** -0.5, nw1, False, "silu", 1e-5, lS, *where, a_off=loffs[4], a2=a2,
+                                                  a2_bias=ab, tau=16.0), iters=10, warm=2)
+        t_l = _timed(lambda: ops.linear_attention(lp, loffs[:4], LH, LD, LE, 1.0, nwa, True, "sigmoid", 1e-5, lS, *where, powers=powers,
+                                                  qkv_silu=True), iters=10, warm=2)
+        if decode:
+            like = f"decode step, {B2} requests (reads and writes {LH * LD * LE * 4 / 1e6:.1f} MB of state per request; like: matrix-memory decode step)"
+            new_kw, old_kw = dict(nbytes=B2 * LH * LD * LE * 8.0), dict(nbytes=B2 * MH * MD * ME * 8.0)
+        else:
+            like = (f"over {B} x {L} tokens, {LH} heads of {LD} x {LE} (priced like the recurrence it is: 4 flop per element of S and token on the vector "
+                    f"units; like: matrix memory, {MH} heads of {MD} x {ME})")
+            new_kw = dict(nbytes=T * 2.0 * (sum(lsizes) + LH * LE), vflops=4.0 * T * LH * LD * LE)
+            old_kw = dict(nbytes=T * 2.0 * (width + MH * ME), vflops=4.0 * T * MH * MD * ME)
+        out.append((f"decay per channel: {like}", rec(t_g, **new_kw), rec(t_old, **old_kw)))
+        out.append((f"decay per head: {like}", rec(t_l, **new_kw), rec(t_old, **old_kw)))
+    return out
+
+
+def main_tebalorn(args) -> dict:
+    from semi_pd_amd.models.gukidra import gukidra_uniform
+    from semi_pd_amd.models.penozen import penozen_uniform
+    from semi_pd_amd.models.tebalorn import tebalorn_uniform
+    dev = torch.device("cuda:0")
+    torch.cuda.set_device(dev)
+    names = [n for n in (getattr(args, "arch_sizes", "") or ",".join(TEBALORN_SIZES)).split(",") if n]
+    result = {"what": "Tebalorn next to Gukidra (dense) and Penozen (mixture) at equal layer sizes", "dtype": "bf16", "data": "synthetic",
+              "models": {}, "kernels": {}}
+    for name in names:
+        s, gs, pz = TEBALORN_SIZES[name], GUKIDRA_SIZES[name], PENOZEN_SIZES[name]
+        result["kernels"][name] = [
+            {"kernel": what, "tebalorn": new, "like": old,
+             "roofline_fraction_ratio": round(new["of_roofline"] / max(old["of_roofline"], 1e-9), 2)}
+            for what, new, old in _tebalorn_kernel_pairs(s, gs, dev)]
+
+        def cfg(pattern):
+            return tebalorn_uniform(s["vocab"], s["hidden"], pattern, s["ff"], s["heads"], s["kv"], s["dim"], s["dim"], s["chunk"], s["lheads"],
+                                    s["ldim"], s["lvdim"], s["side"], s["experts"], s["top"], s["ff"] // 2 // s["top"], s["ff"] // 2)
+
+        gcfg = gukidra_uniform(gs["vocab"], gs["hidden"], "amsm", gs["ff"], gs["heads"], gs["kv"], gs["dim"], gs["dim"], gs["window"], gs["pool"],
+                               gs["mheads"], gs["mdim"], gs["mvdim"])
+        pcfg = penozen_uniform(pz["vocab"], pz["hidden"], "adad", pz["heads"], pz["dim"], pz["rot"], pz["vdim"], pz["rank"], pz["dheads"],
+                               pz["kv"], pz["kdim"], pz["dvdim"], pz["experts"], pz["top"], pz["ff"] // pz["top"])
+        result["models"][name] = {
+            "layers": 4,
+            "tebalorn": _model_throughput(cfg("agal"), 2048, 4, 32, 1100, 20),
+            "gukidra": _model_throughput(gcfg, 2048, 4, 32, 1100, 20),
+            "tebalorn_mixture": _model_throughput(cfg("AGAL"), 2048, 4, 32, 1100, 20),
+            "penozen_mixture": _model_throughput(pcfg, 2048, 4, 32, 1100, 20)}
+    print(json.dumps(result), flush=True)
+    return result
+
+
 def main(args) -> dict:
+    if getattr(args, "arch_design", "kudirax") == "tebalorn":
+        return main_tebalorn(args)
     if getattr(args, "arch_design", "kudirax") == "gukidra":
         return main_gukidra(args)
     if getattr(args, "arch_design", "kudirax") == "tibenex":
