@@ -18,7 +18,8 @@
 //    Everything in front of S and v is independent of the chunks before it: channel_operands_kernel / head_operands_kernel compute
 //    it for all (chunk, head) at once and lay it down in the order in which matrix operands are held -- 1 KB per 16 x 32 operand, a
 //    lane's 16 bytes at its own place -- and chunk_walk_kernel, a workgroup per (request, head, up to 64 columns of S), goes through
-//    the chunks with S in fp32 accumulators, operands coming straight into registers one chunk ahead.  Decayed q, k, A and S
+//    the chunks with S in fp32 accumulators, operands coming straight into registers one chunk ahead; half of its waves make the
+//    next S while the other half read results out of the one in front.  Decayed q, k, A and S
 //    enter a product as their upper 16 bits plus the bf16 of the rest (about 2^-17 relative); sums are fp32.
 //    Per-channel decays have no common factor to take out of a sum over d, so a chunk is four tiles of 16 tokens: between
 //    tiles the exponents split at a tile's edge into two parts, neither above 0; inside a tile they split at its middle as long as
@@ -130,15 +131,16 @@ __device__ __forceinline__ void silu8(Frag16& f) {
   float x[8];
   widen8(f, x);
 #pragma unroll
-  for (int u = 0; u < 8; ++u) x[u] = x[u] / (1.0f + __builtin_amdgcn_exp2f(-x[u] * kLinLog2e));
+  for (int u = 0; u < 8; ++u) x[u] *= __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-x[u] * kLinLog2e));
 #pragma unroll
   for (int u = 0; u < 4; ++u) f.w[u] = pack2<bf16_t>(x[2 * u], x[2 * u + 1]);
 }
 
 // ---------------------------------------------------------------------------------- operands of a chunk
 // Per (chunk, head), in KB: decayed queries [4 tiles][ND][hi, lo] | decayed keys, transposed [2 ND tiles of d][2][hi, lo] |
-// A [4 tiles of queries][2][hi, lo].  The 32 tokens of step s of an operand over tokens are, for lanes of group g: 32 s + 4 g .. + 3,
-// then 32 s + 16 + 4 g .. + 3.
+// A [4 tiles of queries][2][hi, lo].  An operand's 32 summed-over elements -- tokens of step s, channels of step kk -- are, for
+// lanes of group g: 32 s + 4 g .. + 3, then 32 s + 16 + 4 g .. + 3: how the rows of two neighbouring 16-row results lie in a
+// lane, so results become operands without changing lanes.
 __host__ __device__ constexpr int lin_q_frag(int nd, int tile, int kk) { return (tile * nd + kk) * 2; }
 __host__ __device__ constexpr int lin_k_frag(int nd, int dt, int s) { return 8 * nd + (dt * 2 + s) * 2; }
 __host__ __device__ constexpr int lin_a_frag(int nd, int tile, int s) { return 16 * nd + (tile * 2 + s) * 2; }
@@ -152,10 +154,22 @@ __device__ __forceinline__ uint4 get_frag(const uint8_t* base, int idx) {
   return *reinterpret_cast<const uint4*>(base + (int64_t)idx * 1024 + (threadIdx.x & 63) * 16);
 }
 
-// the transposed operand [16 rows d][32 tokens] of an LDS tile of token rows
-template <int STRIDE> __device__ __forceinline__ Frag16 transposed(const uint8_t* tile, int s, int col16) {
+// 8 of the 32 elements of a step from a row of memory, in the order above (n a multiple of 4: elements from n on are zero)
+__device__ __forceinline__ Frag16 two_pieces(const bf16_t* row, int first, int n) {
+  const int g = (threadIdx.x & 63) >> 4, d0 = first + 4 * g, d1 = d0 + 16;
+  uint2 a = {0u, 0u}, b = {0u, 0u};
+  if (d0 < n) a = *reinterpret_cast<const uint2*>(row + d0);
+  if (d1 < n) b = *reinterpret_cast<const uint2*>(row + d1);
+  Frag16 f;
+  f.u = uint4{a.x, a.y, b.x, b.y};
+  return f;
+}
+
+// the transposed operand [16 rows][32 tokens] of an LDS tile of token rows; PERMUTED: the rows' elements lie in the order above
+template <int STRIDE, bool PERMUTED> __device__ __forceinline__ Frag16 transposed(const uint8_t* tile, int s, int col16) {
   const int lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
-  const uint8_t* row = tile + (32 * s + 4 * g + (r >> 2)) * STRIDE + (r & 3) * 8 + col16 * 32;
+  const uint8_t* row = tile + (32 * s + 4 * g + (r >> 2)) * STRIDE +
+                       (PERMUTED ? (r & 3) * 16 + (col16 & 1) * 8 + (col16 >> 1) * 64 : (r & 3) * 8 + col16 * 32);
   Frag16 f;
   f.s[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)row);
   f.s[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(row + 16 * STRIDE));
@@ -178,203 +192,190 @@ __device__ __forceinline__ void put_weights(uint8_t* base, int nd, int tile, con
   }
 }
 
-constexpr int kLinRankBlock = 16;
-template <int ND> constexpr size_t channel_lds() {
-  constexpr size_t c = (size_t)kLinChunk * (32 * ND + 4) * sizeof(float), k = 2 * (size_t)kLinChunk * lin_row(ND);
-  return (c > k ? c : k) + 4 * 32 * ND * sizeof(float) + kLinRankBlock * kLinChunk * sizeof(float);
+// keys of the chunk in LDS (upper and lower parts) -> transposed operands, ND / 2 tiles of d per wave
+template <int ND> __device__ __forceinline__ void put_keys(uint8_t* base, const uint8_t* kh, const uint8_t* kl) {
+  const int wave = threadIdx.x >> 6;
+#pragma unroll
+  for (int i = 0; i < ND / 2; ++i) {
+    const int dt = (ND / 2) * wave + i;
+#pragma unroll
+    for (int s = 0; s < 2; ++s) {
+      put_frag(base, lin_k_frag(ND, dt, s), transposed<lin_row(ND), true>(kh, s, dt));
+      put_frag(base, lin_k_frag(ND, dt, s) + 1, transposed<lin_row(ND), true>(kl, s, dt));
+    }
+  }
 }
 
-template <int ND>          // key sizes up to 32 ND; wave = tile of 16 tokens
+template <int CTRL> __device__ __forceinline__ float dpp(float x) {       // row operations inside 16 lanes, 0 where nothing comes in
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), CTRL, 0xf, 0xf, false));
+}
+__device__ __forceinline__ float sum_up_to(float x) {                     // inclusive running sum over 16 lanes
+  x += dpp<0x111>(x);
+  x += dpp<0x112>(x);
+  x += dpp<0x114>(x);
+  return x + dpp<0x118>(x);
+}
+template <int LANE> __device__ __forceinline__ float of_lane(float x) { return dpp<0x150 + LANE>(x); }      // lane LANE of the 16 (row_newbcast)
+
+template <int ND> constexpr size_t channel_lds() { return 2 * (size_t)kLinChunk * lin_row(ND) + 4 * 32 * ND * sizeof(float); }
+
+template <int ND>          // key sizes up to 32 ND; wave = tile of 16 tokens, lane r of 16 = token
 __global__ void __launch_bounds__(256, 2) channel_operands_kernel(LinArgs a) {
   extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-  constexpr int DP = 32 * ND, CS = DP + 4, RS = lin_row(ND), ITEMS = ND / 2;
-  constexpr size_t kFirst = (size_t)kLinChunk * CS * 4 > 2 * (size_t)kLinChunk * RS ? (size_t)kLinChunk * CS * 4 : 2 * (size_t)kLinChunk * RS;
-  float* c_lds = reinterpret_cast<float*>(lds);                         // running sums inside a tile [64][CS]; later the keys
+  constexpr int DP = 32 * ND, RS = lin_row(ND);
   uint8_t* kh = lds;                                                    // keys, upper and lower parts [64][RS]
   uint8_t* kl = lds + kLinChunk * RS;
-  float* tot = reinterpret_cast<float*>(lds + kFirst);                  // sums over whole tiles [4][DP]
-  float* a1 = tot + 4 * DP;                                             // [rank block][64 tokens]
+  float* loss = reinterpret_cast<float*>(lds + 2 * kLinChunk * RS);     // what a channel keeps over a whole tile [4][DP], in the operands' order
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
-  const int h = blockIdx.y, D = a.D;
+  const int h = blockIdx.y, D = a.D, rank = a.rank;
   int b;
   int64_t c;
   if (!find_chunk(a, blockIdx.x, b, c)) return;
   const int64_t c0 = c * kLinChunk;
   const int cnt = (int)(a.q_len[b] - c0 < kLinChunk ? a.q_len[b] - c0 : kLinChunk);
-  const bf16_t* p = (const bf16_t*)a.p + (a.q_start[b] + c0) * a.ld;
-  uint8_t* out = a.frags + ((int64_t)blockIdx.x * a.H + h) * lin_frags(ND) * 1024;
-
-  // log2 decays of (tile s, channel d) = item, and their running sums
-  float z[ITEMS][16];
-#pragma unroll
-  for (int i = 0; i < ITEMS; ++i)
-#pragma unroll
-    for (int u = 0; u < 16; ++u) z[i][u] = 0.f;
-  const bf16_t* a2 = (const bf16_t*)a.a2 + (int64_t)h * D * a.rank;
-  for (int r0 = 0; r0 < a.rank; r0 += kLinRankBlock) {
-    const int nr = a.rank - r0 < kLinRankBlock ? a.rank - r0 : kLinRankBlock;
-    if (r0) __syncthreads();
-    for (int i = tid; i < kLinRankBlock * kLinChunk; i += 256) {
-      const int t = i / kLinRankBlock, rr = i % kLinRankBlock;
-      a1[rr * kLinChunk + t] = rr < nr ? Elem<bf16_t>::to_f(p[(int64_t)(t < cnt ? t : cnt - 1) * a.ld + a.a_off + r0 + rr]) : 0.f;
-    }
-    __syncthreads();
-#pragma unroll
-    for (int i = 0; i < ITEMS; ++i) {
-      const int it = tid + 256 * i, s = it / DP, d = it % DP;
-      const bf16_t* w = a2 + (int64_t)(d < D ? d : 0) * a.rank + r0;
-      for (int rr = 0; rr < nr; ++rr) {
-        const float x = Elem<bf16_t>::to_f(w[rr]);
-        const float4* row = reinterpret_cast<const float4*>(a1 + rr * kLinChunk + 16 * s);
-#pragma unroll
-        for (int u = 0; u < 4; ++u) {
-          const float4 y = row[u];
-          z[i][4 * u] += x * y.x;
-          z[i][4 * u + 1] += x * y.y;
-          z[i][4 * u + 2] += x * y.z;
-          z[i][4 * u + 3] += x * y.w;
-        }
-      }
-    }
-  }
-#pragma unroll
-  for (int i = 0; i < ITEMS; ++i) {
-    const int it = tid + 256 * i, s = it / DP, d = it % DP;
-    const float bias = d < D ? a.a2_bias[h * D + d] : 0.f;
-    float run = 0.f;
-#pragma unroll
-    for (int u = 0; u < 16; ++u) {
-      if (d < D && 16 * s + u < cnt) run += log2_decay(z[i][u] + bias, a.inv_tau);
-      c_lds[(16 * s + u) * CS + d] = run;
-    }
-    tot[s * DP + d] = run;
-  }
-  __syncthreads();
-
-  if (tid < DP) a.keep[((int64_t)blockIdx.x * a.H + h) * DP + tid] =
-      __builtin_amdgcn_exp2f((tot[tid] + tot[DP + tid]) + (tot[2 * DP + tid] + tot[3 * DP + tid]));
-
-  // this lane's query and key: token 16 wave + r, elements 32 kk + 8 g ..
   const int row = 16 * wave + r;
-  const bf16_t* pr = p + (int64_t)(row < cnt ? row : cnt - 1) * a.ld + (int64_t)h * D;
-  bool gentle = true;                    // no channel loses more than 2^100 over this wave's tile
-  for (int d = lane; d < DP; d += 64) gentle = gentle && tot[wave * DP + d] > -100.f;
-  gentle = __all(gentle);
-  float q8[ND][8], k8[ND][8];
-  f32x4 own = {0.f, 0.f, 0.f, 0.f};
+  const bf16_t* pr = (const bf16_t*)a.p + (a.q_start[b] + c0 + (row < cnt ? row : cnt - 1)) * a.ld;
+  uint8_t* out = a.frags + ((int64_t)blockIdx.x * a.H + h) * lin_frags(ND) * 1024;
+  const bf16_t* a2 = (const bf16_t*)a.a2 + (int64_t)h * D * rank;
+  const bool wide = rank % 4 == 0 && (a.a_off & 3) == 0 && ((uintptr_t)a.a2 & 7) == 0;
+  auto rank_piece = [&](const bf16_t* src, int first) {                 // 32 elements of a row of A1 h or A2
+    if (wide) return two_pieces(src, first, rank);
+    Frag16 f;
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int i = first + 4 * g + (u & 3) + (u >> 2) * 16;
+      f.e[u] = i < rank ? src[i].v : (uint16_t)0;
+    }
+    return f;
+  };
+  const Frag16 a1 = rank_piece(pr + a.a_off, 0);
+
+  float q8[ND][8], k8[ND][8];              // queries from their tile's start, keys to their tile's end
+  f32x4 own = {0.f, 0.f, 0.f, 0.f};        // A inside the tile: key 4 g + i, query r
 #pragma unroll
   for (int kk = 0; kk < ND; ++kk) {
-    const int d0 = 32 * kk + 8 * g;
-    Frag16 qf, kf;
-    qf.u = kf.u = uint4{0u, 0u, 0u, 0u};
-    if (d0 < D) {
-      qf.u = *reinterpret_cast<const uint4*>(pr + a.q_off + d0);
-      if (row < cnt) kf.u = *reinterpret_cast<const uint4*>(pr + a.k_off + d0);
+    // running sums of the log2 decays: rows = channels 32 kk + 16 half + 4 g + i, column = this lane's token
+    float cs[8], q[8], k[8];
+#pragma unroll
+    for (int half = 0; half < 2; ++half) {
+      const int dr = 32 * kk + 16 * half + r, dz = 32 * kk + 16 * half + 4 * g;
+      const bf16_t* w = a2 + (int64_t)(dr < D ? dr : 0) * rank;
+      float bias[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) bias[i] = dz < D ? a.a2_bias[h * D + dz + i] : 0.f;
+      f32x4 z = {0.f, 0.f, 0.f, 0.f};
+      z = mma16<bf16_t>(rank_piece(w, 0), a1, z);
+      for (int r0 = 32; r0 < rank; r0 += 32) z = mma16<bf16_t>(rank_piece(w, r0), rank_piece(pr + a.a_off, r0), z);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const bool there = row < cnt && dz < D;
+        const float x = there ? log2_decay(z[i] + bias[i], a.inv_tau) : 0.f;
+        cs[4 * half + i] = sum_up_to(x);
+      }
     }
+    Frag16 qf = two_pieces(pr + a.q_off + (int64_t)h * D, 32 * kk, D), kf = two_pieces(pr + a.k_off + (int64_t)h * D, 32 * kk, row < cnt ? D : 0);
     if (a.act) {
       silu8(qf);
       silu8(kf);
     }
-    float q[8], k[8], cs[8], before[8], total[8];
     widen8(qf, q);
     widen8(kf, k);
-    auto read8 = [&](const float* src, float (&x)[8]) {
-      const float4 lo = *reinterpret_cast<const float4*>(src), hi = *reinterpret_cast<const float4*>(src + 4);
-      x[0] = lo.x; x[1] = lo.y; x[2] = lo.z; x[3] = lo.w; x[4] = hi.x; x[5] = hi.y; x[6] = hi.z; x[7] = hi.w;
-    };
-    read8(c_lds + row * CS + d0, cs);
-    read8(tot + wave * DP + d0, total);
+    float total[8];
+    bool gentle = true;                    // none of these channels loses more than 2^100 over the tile
 #pragma unroll
-    for (int u = 0; u < 8; ++u) before[u] = 0.f;
-    for (int s = 0; s < wave; ++s) {
-      float t[8];
-      read8(tot + s * DP + d0, t);
-#pragma unroll
-      for (int u = 0; u < 8; ++u) before[u] += t[u];
+    for (int u = 0; u < 8; ++u) {
+      total[u] = of_lane<15>(cs[u]);
+      gentle = gentle && total[u] > -100.f;
     }
-    float x[8];
-    Frag16 hi, lo;
+    if (r == 0) {
+      float* t = loss + wave * DP + 32 * kk + 8 * g;
 #pragma unroll
-    for (int u = 0; u < 8; ++u) x[u] = q[u] * __builtin_amdgcn_exp2f(before[u] + cs[u]);
-    hi_lo8(x, hi, lo);
-    put_frag(out, lin_q_frag(ND, wave, kk), hi);
-    put_frag(out, lin_q_frag(ND, wave, kk) + 1, lo);
-    if (gentle) {                        // the tile's own pairs: both sides relative to the tile's eighth token
-      float mid[8];
-      read8(c_lds + (16 * wave + 7) * CS + d0, mid);
-      Frag16 ah, al;
+      for (int u = 0; u < 8; ++u) t[u] = __builtin_amdgcn_exp2f(total[u]);
+    }
+    if (__all(gentle)) {                   // the tile's own pairs: both sides relative to the tile's eighth token
+      Frag16 qh, ql, ah, al;
 #pragma unroll
-      for (int u = 0; u < 8; ++u) x[u] = q[u] * __builtin_amdgcn_exp2f(cs[u] - mid[u]);
-      hi_lo8(x, hi, lo);
-#pragma unroll
-      for (int u = 0; u < 8; ++u) x[u] = k[u] * __builtin_amdgcn_exp2f(mid[u] - cs[u]);
-      hi_lo8(x, ah, al);
-      own = mma16<bf16_t>(ah, hi, own);
-      own = mma16<bf16_t>(al, hi, own);
-      own = mma16<bf16_t>(ah, lo, own);
-    } else {                             // pair by pair; the pairs' sums over d are completed across the lane groups below
+      for (int u = 0; u < 8; ++u) {
+        const float mid = of_lane<7>(cs[u]), e = __builtin_amdgcn_exp2f(cs[u] - mid);
+        q[u] *= e;
+        k[u] *= __builtin_amdgcn_rcpf(e);
+        q8[kk][u] = q[u] * __builtin_amdgcn_exp2f(mid);
+        k8[kk][u] = k[u] * __builtin_amdgcn_exp2f(total[u] - mid);
+      }
+      hi_lo8(q, qh, ql);
+      hi_lo8(k, ah, al);
+      own = mma16<bf16_t>(ah, qh, own);
+      own = mma16<bf16_t>(al, qh, own);
+      own = mma16<bf16_t>(ah, ql, own);
+    } else {                               // pair by pair
 #pragma unroll 1
       for (int j = 0; j < 16; ++j) {
-        const int kr = 16 * wave + j;
-        float cj[8], part = 0.f, kj[8];
-        read8(c_lds + kr * CS + d0, cj);
-        Frag16 f;
-        f.u = uint4{0u, 0u, 0u, 0u};
-        if (d0 < D && kr < cnt) f.u = *reinterpret_cast<const uint4*>(p + (int64_t)kr * a.ld + (int64_t)h * D + a.k_off + d0);
-        if (a.act) silu8(f);
-        widen8(f, kj);
+        float part = 0.f;
 #pragma unroll
-        for (int u = 0; u < 8; ++u) part += q[u] * kj[u] * __builtin_amdgcn_exp2f(fminf(cs[u] - cj[u], 0.f));
+        for (int u = 0; u < 8; ++u) {
+          const float cj = __shfl(cs[u], (lane & 48) | j, 64), kj = __shfl(k[u], (lane & 48) | j, 64);
+          part += q[u] * kj * __builtin_amdgcn_exp2f(fminf(cs[u] - cj, 0.f));
+        }
         part += __shfl_xor(part, 16, 64);
         part += __shfl_xor(part, 32, 64);
 #pragma unroll
         for (int i = 0; i < 4; ++i)
           if (4 * g + i == j) own[i] += part;
       }
-    }
 #pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      q8[kk][u] = q[u] * __builtin_amdgcn_exp2f(cs[u]);
-      k8[kk][u] = k[u] * __builtin_amdgcn_exp2f(total[u] - cs[u]);
+      for (int u = 0; u < 8; ++u) {
+        q8[kk][u] = q[u] * __builtin_amdgcn_exp2f(cs[u]);
+        k8[kk][u] = k[u] * __builtin_amdgcn_exp2f(total[u] - cs[u]);
+      }
     }
+    Frag16 hi, lo;
+    hi_lo8(k8[kk], hi, lo);
+    *reinterpret_cast<uint4*>(kh + row * RS + (32 * kk + 8 * g) * 2) = hi.u;
+    *reinterpret_cast<uint4*>(kl + row * RS + (32 * kk + 8 * g) * 2) = lo.u;
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i) own[i] = 4 * g + i <= r ? own[i] : 0.f;
-  __syncthreads();                       // the running sums have been read by everyone: keys take their place
-  auto lay_keys = [&]() {
-#pragma unroll
-    for (int kk = 0; kk < ND; ++kk) {
-      Frag16 hi, lo;
-      hi_lo8(k8[kk], hi, lo);
-      *reinterpret_cast<uint4*>(kh + row * RS + (32 * kk + 8 * g) * 2) = hi.u;
-      *reinterpret_cast<uint4*>(kl + row * RS + (32 * kk + 8 * g) * 2) = lo.u;
-    }
-  };
-  lay_keys();
   __syncthreads();
-  // tiles in front: keys relative to their tile's end, queries to the end of that tile
-  f32x4 back[3];                         // tile wave - 1 - x
+  if (tid < DP) {
+    const int p32 = tid & 31, d = (tid & ~31) + ((p32 >> 2) & 1) * 16 + (p32 >> 3) * 4 + (p32 & 3);
+    a.keep[((int64_t)blockIdx.x * a.H + h) * DP + d] = (loss[tid] * loss[DP + tid]) * (loss[2 * DP + tid] * loss[3 * DP + tid]);
+  }
+  auto read8 = [&](int tile, int kk, float (&x)[8]) {
+    const float* src = loss + tile * DP + 32 * kk + 8 * g;
+    const float4 lo = *reinterpret_cast<const float4*>(src), hi = *reinterpret_cast<const float4*>(src + 4);
+    x[0] = lo.x; x[1] = lo.y; x[2] = lo.z; x[3] = lo.w; x[4] = hi.x; x[5] = hi.y; x[6] = hi.z; x[7] = hi.w;
+  };
+  // tiles in front, from the nearest on: keys relative to their tile's end, queries brought to the end of that tile, and past the
+  // first tile to the chunk's start
+  f32x4 back[3];                           // tile wave - 1 - x
 #pragma unroll
   for (int x = 0; x < 3; ++x) back[x] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int kk = 0; kk < ND; ++kk) {
-    const int d0 = 32 * kk + 8 * g;
+    Frag16 hi, lo;
+    float t[8];
 #pragma unroll
     for (int x = 0; x < 3; ++x) {
       const int J = wave - 1 - x;
       if (J < 0) break;
-      if (x > 0) {
-        const float* t = tot + (J + 1) * DP + d0;
-#pragma unroll
-        for (int u = 0; u < 8; ++u) q8[kk][u] *= __builtin_amdgcn_exp2f(t[u]);
-      }
-      Frag16 hi, lo, ah, al;
+      Frag16 ah, al;
+      ah.u = *reinterpret_cast<const uint4*>(kh + (16 * J + r) * RS + (32 * kk + 8 * g) * 2);
+      al.u = *reinterpret_cast<const uint4*>(kl + (16 * J + r) * RS + (32 * kk + 8 * g) * 2);
       hi_lo8(q8[kk], hi, lo);
-      ah.u = *reinterpret_cast<const uint4*>(kh + (16 * J + r) * RS + d0 * 2);
-      al.u = *reinterpret_cast<const uint4*>(kl + (16 * J + r) * RS + d0 * 2);
       back[x] = mma16<bf16_t>(ah, hi, back[x]);
       back[x] = mma16<bf16_t>(al, hi, back[x]);
       back[x] = mma16<bf16_t>(ah, lo, back[x]);
+      read8(J, kk, t);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) q8[kk][u] *= t[u];
+    }
+    hi_lo8(q8[kk], hi, lo);
+    put_frag(out, lin_q_frag(ND, wave, kk), hi);
+    put_frag(out, lin_q_frag(ND, wave, kk) + 1, lo);
+    for (int s = wave + 1; s < 4; ++s) {   // keys to the chunk's end
+      read8(s, kk, t);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) k8[kk][u] *= t[u];
     }
   }
   f32x4 w[4];
@@ -387,31 +388,16 @@ __global__ void __launch_bounds__(256, 2) channel_operands_kernel(LinArgs a) {
       if (kt == wave - 1 - x) w[kt] = back[x];
   }
   put_weights(out, ND, wave, w);
-  // keys relative to the chunk's end
+  __syncthreads();
 #pragma unroll
   for (int kk = 0; kk < ND; ++kk) {
-    const int d0 = 32 * kk + 8 * g;
-    float after[8];
-#pragma unroll
-    for (int u = 0; u < 8; ++u) after[u] = 0.f;
-    for (int s = wave + 1; s < 4; ++s)
-#pragma unroll
-      for (int u = 0; u < 8; ++u) after[u] += tot[s * DP + d0 + u];
-#pragma unroll
-    for (int u = 0; u < 8; ++u) k8[kk][u] *= __builtin_amdgcn_exp2f(after[u]);
+    Frag16 hi, lo;
+    hi_lo8(k8[kk], hi, lo);
+    *reinterpret_cast<uint4*>(kh + row * RS + (32 * kk + 8 * g) * 2) = hi.u;
+    *reinterpret_cast<uint4*>(kl + row * RS + (32 * kk + 8 * g) * 2) = lo.u;
   }
   __syncthreads();
-  lay_keys();
-  __syncthreads();
-#pragma unroll
-  for (int i = 0; i < ND / 2; ++i) {
-    const int dt = (ND / 2) * wave + i;
-#pragma unroll
-    for (int s = 0; s < 2; ++s) {
-      put_frag(out, lin_k_frag(ND, dt, s), transposed<RS>(kh, s, dt));
-      put_frag(out, lin_k_frag(ND, dt, s) + 1, transposed<RS>(kl, s, dt));
-    }
-  }
+  put_keys<ND>(out, kh, kl);
 }
 
 template <int ND>          // one decay per head: it factors out of the sum over d
@@ -428,20 +414,15 @@ __global__ void __launch_bounds__(256, 2) head_operands_kernel(LinArgs a) {
   if (!find_chunk(a, blockIdx.x, b, c)) return;
   const int64_t c0 = c * kLinChunk;
   const int cnt = (int)(a.q_len[b] - c0 < kLinChunk ? a.q_len[b] - c0 : kLinChunk);
-  const bf16_t* p = (const bf16_t*)a.p + (a.q_start[b] + c0) * a.ld;
   uint8_t* out = a.frags + ((int64_t)blockIdx.x * a.H + h) * lin_frags(ND) * 1024;
   if (tid <= kLinChunk) pw[tid] = a.powers[h * (kLinChunk + 1) + tid];
   const int row = 16 * wave + r;
-  const bf16_t* pr = p + (int64_t)(row < cnt ? row : cnt - 1) * a.ld + (int64_t)h * D;
+  const bf16_t* pr = (const bf16_t*)a.p + (a.q_start[b] + c0 + (row < cnt ? row : cnt - 1)) * a.ld + (int64_t)h * D;
   Frag16 qf[ND], kf[ND];
 #pragma unroll
   for (int kk = 0; kk < ND; ++kk) {
-    const int d0 = 32 * kk + 8 * g;
-    qf[kk].u = kf[kk].u = uint4{0u, 0u, 0u, 0u};
-    if (d0 < D) {
-      qf[kk].u = *reinterpret_cast<const uint4*>(pr + a.q_off + d0);
-      if (row < cnt) kf[kk].u = *reinterpret_cast<const uint4*>(pr + a.k_off + d0);
-    }
+    qf[kk] = two_pieces(pr + a.q_off, 32 * kk, D);
+    kf[kk] = two_pieces(pr + a.k_off, 32 * kk, row < cnt ? D : 0);
   }
   if (a.act) {
 #pragma unroll
@@ -497,33 +478,27 @@ __global__ void __launch_bounds__(256, 2) head_operands_kernel(LinArgs a) {
     *reinterpret_cast<uint4*>(kl + row * RS + (32 * kk + 8 * g) * 2) = lo.u;
   }
   __syncthreads();
-#pragma unroll
-  for (int i = 0; i < ND / 2; ++i) {
-    const int dt = (ND / 2) * wave + i;
-#pragma unroll
-    for (int s = 0; s < 2; ++s) {
-      put_frag(out, lin_k_frag(ND, dt, s), transposed<RS>(kh, s, dt));
-      put_frag(out, lin_k_frag(ND, dt, s) + 1, transposed<RS>(kl, s, dt));
-    }
-  }
+  put_keys<ND>(out, kh, kl);
 }
 
 // ---------------------------------------------------------------------------------- the walk over a request's chunks
+// Eight waves with two jobs.  Waves 4 .. 7 carry S in fp32 accumulators from chunk to chunk: S <- diag(e^(b_last)) S + K^T V, then S
+// as upper and lower bf16 parts into LDS; they also bring the chunk's values there.  Waves 0 .. 3, one per 16 queries, turn the S
+// that the chunk found and its values into results.  S and the values have two places each, so while results of a chunk are
+// computed the next S is already being made, with one barrier per chunk; both jobs' operands come from memory straight into
+// registers, one chunk ahead.
 template <int EC> constexpr int lin_v_row() { return EC * 32 + 32; }
-template <int ND, int EC> constexpr size_t walk_lds() { return 2 * (size_t)(16 * EC) * lin_row(ND) + (size_t)kLinChunk * lin_v_row<EC>(); }
+template <int ND, int EC> constexpr size_t walk_lds() { return 4 * (size_t)(16 * EC) * lin_row(ND) + 2 * (size_t)kLinChunk * lin_v_row<EC>(); }
 
-template <int ND, int EC>          // key sizes up to 32 ND; 16 EC columns of S per workgroup of eight waves
+template <int ND, int EC>          // key sizes up to 32 ND; 16 EC columns of S per workgroup
 __global__ void __launch_bounds__(512, 2) chunk_walk_kernel(LinArgs a) {
   extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
   constexpr int RS = lin_row(ND), VS = lin_v_row<EC>(), DP = 32 * ND, COLS = 16 * EC;
-  // tiles of S of a wave: DTW tiles of d from dt0, ETW tiles of columns from et0; tiles of the result: ETO from eto0, queries qt
-  constexpr int DTW = ND >= 4 ? ND / 4 : 1, ETW = ND >= 4 ? EC : EC / 2, ETO = EC / 2;
-  uint8_t* s_hi = lds;
-  uint8_t* s_lo = lds + COLS * RS;
-  uint8_t* v_lds = lds + 2 * COLS * RS;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, g = lane >> 4;
-  const int qt = wave & 3, eto0 = (wave >> 2) * ETO;
-  const int dt0 = ND >= 4 ? wave * DTW : wave >> 1, et0 = ND >= 4 ? 0 : (wave & 1) * ETW;
+  constexpr int S_PART = COLS * RS, S_BUF = 2 * S_PART, V_BUF = kLinChunk * VS;
+  uint8_t* s_lds = lds;                                                  // [2][upper, lower][COLS][RS]
+  uint8_t* v_lds = lds + 2 * S_BUF;                                      // [2][64][VS]
+  const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int H = a.H, D = a.D, E = a.E;
   const int slices = (E + COLS - 1) / COLS;
   // consecutive workgroup ids go round the eight XCDs: an XCD takes a contiguous range of items, so the slices of a head --
@@ -533,50 +508,146 @@ __global__ void __launch_bounds__(512, 2) chunk_walk_kernel(LinArgs a) {
   const int sl = (int)(item % slices), h = (int)(item / slices % H), b = (int)(item / slices / H);
   int64_t t0, n, first_pos;
   if (!linear_rows(a, b, t0, n, first_pos)) return;
-  const bool fresh = first_pos == 0;
   const int e0 = sl * COLS;
   const int64_t chunk0 = chunks_before(a, b);
-  const bf16_t* vp = (const bf16_t*)a.p + t0 * a.ld + a.v_off + (int64_t)h * E + e0;
-  float* work = a.work + t0 * a.wld + (int64_t)h * E + e0;
-  float* S = a.state + a.state_indices[b] * a.state_ld + (int64_t)h * D * E + e0;
-  const int64_t frag_step = (int64_t)H * lin_frags(ND) * 1024, keep_step = (int64_t)H * DP;
+  const int chunks = (int)((n + kLinChunk - 1) / kLinChunk);             // every wave passes 1 barrier per chunk
+  const int64_t frag_step = (int64_t)H * lin_frags(ND) * 1024;
   const uint8_t* fr = a.frags + (chunk0 * H + h) * (int64_t)lin_frags(ND) * 1024;
-  const float* keep = a.keep + (chunk0 * H + h) * DP;
 
-  f32x4 acc[DTW][ETW];               // rows d = 16 (dt0 + dt) + 4 g + i, column e0 + 16 (et0 + et) + r
+  if (wave < 4) {
+    // ---- results of queries 16 wave + r, all columns
+    const int qt = wave;
+    float* work = a.work + (t0 + 16 * qt + r) * a.wld + (int64_t)h * E + e0;
+    Frag16 qf[ND][2], wf[2][2];
+    auto fetch_q = [&](const uint8_t* f) {
+#pragma unroll
+      for (int kk = 0; kk < ND; ++kk) {
+        qf[kk][0].u = get_frag(f, lin_q_frag(ND, qt, kk));
+        qf[kk][1].u = get_frag(f, lin_q_frag(ND, qt, kk) + 1);
+      }
+    };
+    auto fetch_w = [&](const uint8_t* f) {
+#pragma unroll
+      for (int s = 0; s < 2; ++s) {
+        if (2 * s > qt) break;
+        wf[s][0].u = get_frag(f, lin_a_frag(ND, qt, s));
+        wf[s][1].u = get_frag(f, lin_a_frag(ND, qt, s) + 1);
+      }
+    };
+    fetch_q(fr);
+    fetch_w(fr);
+    for (int c = 0; c < chunks; ++c) {
+      const int64_t left = n - (int64_t)c * kLinChunk - 16 * qt;         // rows of this tile that are there
+      const bool more = c + 1 < chunks;
+      const uint8_t* s_hi = s_lds + (c & 1) * S_BUF;
+      const uint8_t* s_lo = s_hi + S_PART;
+      const uint8_t* v_in = v_lds + (c & 1) * V_BUF;
+      fr += frag_step;
+      __syncthreads();
+      f32x4 o[EC];
+#pragma unroll
+      for (int et = 0; et < EC; ++et) o[et] = f32x4{0.f, 0.f, 0.f, 0.f};
+      // the operands of the next 32 elements are on their way out of LDS during a product
+      Frag16 sa[2][EC][2];
+      auto load = [&](int kk, Frag16 (&x)[EC][2]) {
+#pragma unroll
+        for (int et = 0; et < EC; ++et) {
+          const int off = (16 * et + r) * RS + g * 16 + kk * 64;
+          x[et][0].u = *reinterpret_cast<const uint4*>(s_hi + off);
+          x[et][1].u = *reinterpret_cast<const uint4*>(s_lo + off);
+        }
+      };
+      load(0, sa[0]);
+#pragma unroll
+      for (int kk = 0; kk < ND; ++kk) {
+        if (kk + 1 < ND) load(kk + 1, sa[(kk + 1) & 1]);
+        __builtin_amdgcn_sched_barrier(0);
+        Frag16(&x)[EC][2] = sa[kk & 1];
+#pragma unroll
+        for (int et = 0; et < EC; ++et) o[et] = mma16<bf16_t>(x[et][0], qf[kk][0], o[et]);
+#pragma unroll
+        for (int et = 0; et < EC; ++et) o[et] = mma16<bf16_t>(x[et][1], qf[kk][0], o[et]);
+#pragma unroll
+        for (int et = 0; et < EC; ++et) o[et] = mma16<bf16_t>(x[et][0], qf[kk][1], o[et]);
+        __builtin_amdgcn_sched_barrier(0);
+      }
+      if (more) fetch_q(fr);
+      // the chunk's own tokens
+#pragma unroll
+      for (int s = 0; s < 2; ++s) {
+        if (2 * s > qt) break;
+        Frag16 v[EC];
+#pragma unroll
+        for (int et = 0; et < EC; ++et) v[et] = transposed<VS, false>(v_in, s, et);
+#pragma unroll
+        for (int et = 0; et < EC; ++et) o[et] = mma16<bf16_t>(v[et], wf[s][0], o[et]);
+#pragma unroll
+        for (int et = 0; et < EC; ++et) o[et] = mma16<bf16_t>(v[et], wf[s][1], o[et]);
+      }
+      if (more) fetch_w(fr);
+      if (r < left) {
+#pragma unroll
+        for (int et = 0; et < EC; ++et) {
+          const int e = 16 * et + 4 * g;
+          if (e0 + e < E) *reinterpret_cast<float4*>(work + e) =
+              float4{o[et][0] * a.q_scale, o[et][1] * a.q_scale, o[et][2] * a.q_scale, o[et][3] * a.q_scale};
+        }
+      }
+      work += kLinChunk * a.wld;
+    }
+    return;
+  }
+
+  // ---- S: rows d = 16 (dt0 + dt) + 4 g + i, column e0 + 16 et + r
+  constexpr int DTW = ND / 2, VP = EC / 2;
+  const int dt0 = (wave - 4) * DTW, vt = tid - 256;
+  const bool fresh = first_pos == 0;
+  float* S = a.state + a.state_indices[b] * a.state_ld + (int64_t)h * D * E + e0;
+  const int64_t keep_step = (int64_t)H * DP;
+  const float* keep = a.keep + (chunk0 * H + h) * DP;
+  const bf16_t* vp = (const bf16_t*)a.p + t0 * a.ld + a.v_off + (int64_t)h * E;
+  f32x4 acc[DTW][EC];
 #pragma unroll
   for (int dt = 0; dt < DTW; ++dt)
 #pragma unroll
-    for (int et = 0; et < ETW; ++et)
+    for (int et = 0; et < EC; ++et)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int d = 16 * (dt0 + dt) + 4 * g + i, e = 16 * (et0 + et) + r;
+        const int d = 16 * (dt0 + dt) + 4 * g + i, e = 16 * et + r;
         acc[dt][et][i] = (!fresh && d < D && e0 + e < E) ? S[(int64_t)d * E + e] : 0.f;
       }
-  // values: a thread moves one 16-byte piece of the chunk's 64 rows (past the end the last row, past E the first columns: finite
-  // numbers that meet zero weights or columns that are not kept)
-  const int v_row = tid / (2 * EC), v_e = (tid % (2 * EC)) * 8;
-  const bool v_mine = v_row < kLinChunk;
-  const int v_col = e0 + v_e < E ? v_e : 0;
-  Frag16 qf[ND][2], kf[DTW][2][2], wf[2][2], vr;
+  Frag16 kf[DTW][2][2], vr[VP];
   float4 kp[DTW];
-  auto fetch_v = [&](int64_t c0) {
-    const int64_t last = n - 1 - c0;
-    if (v_mine) vr.u = *reinterpret_cast<const uint4*>(vp + (c0 + (v_row < last ? v_row : last)) * a.ld + v_col);
-  };
-  auto fetch_q = [&](const uint8_t* f) {
+  // values, in 16-byte pieces (past the end the last row, past E the first columns: finite numbers that meet zero weights or
+  // columns that are not kept)
+  auto fetch_v = [&](int c) {
+    const int64_t base = (int64_t)c * kLinChunk, last = n - 1 - base;
 #pragma unroll
-    for (int kk = 0; kk < ND; ++kk) {
-      qf[kk][0].u = get_frag(f, lin_q_frag(ND, qt, kk));
-      qf[kk][1].u = get_frag(f, lin_q_frag(ND, qt, kk) + 1);
+    for (int i = 0; i < VP; ++i) {
+      const int x = vt + 256 * i, row = x / (2 * EC), e = e0 + (x % (2 * EC)) * 8;
+      vr[i].u = *reinterpret_cast<const uint4*>(vp + (base + (row < last ? row : last)) * a.ld + (e < E ? e : 0));
     }
   };
-  auto fetch_w = [&](const uint8_t* f) {
+  auto lay_v = [&](uint8_t* v_out) {
 #pragma unroll
-    for (int s = 0; s < 2; ++s) {
-      if (2 * s > qt) break;
-      wf[s][0].u = get_frag(f, lin_a_frag(ND, qt, s));
-      wf[s][1].u = get_frag(f, lin_a_frag(ND, qt, s) + 1);
+    for (int i = 0; i < VP; ++i) {
+      const int x = vt + 256 * i;
+      if (a.act) silu8(vr[i]);
+      *reinterpret_cast<uint4*>(v_out + x / (2 * EC) * VS + (x % (2 * EC)) * 16) = vr[i].u;
+    }
+  };
+  auto lay_s = [&](uint8_t* s_out) {
+#pragma unroll
+    for (int dt = 0; dt < DTW; ++dt) {
+      const int at = ((dt0 + dt) >> 1) * 64 + 16 * g + ((dt0 + dt) & 1) * 8;      // in the operands' order
+#pragma unroll
+      for (int et = 0; et < EC; ++et) {
+        uint2 hi, lo;
+        hi_lo(acc[dt][et][0], acc[dt][et][1], hi.x, lo.x);
+        hi_lo(acc[dt][et][2], acc[dt][et][3], hi.y, lo.y);
+        *reinterpret_cast<uint2*>(s_out + (16 * et + r) * RS + at) = hi;
+        *reinterpret_cast<uint2*>(s_out + S_PART + (16 * et + r) * RS + at) = lo;
+      }
     }
   };
   auto fetch_k = [&](const uint8_t* f, const float* kd) {
@@ -591,87 +662,24 @@ __global__ void __launch_bounds__(512, 2) chunk_walk_kernel(LinArgs a) {
     }
   };
   fetch_v(0);
-  fetch_q(fr);
-  fetch_w(fr);
   fetch_k(fr, keep);
-  for (int64_t c0 = 0; c0 < n; c0 += kLinChunk) {
-    const int cnt = (int)(n - c0 < kLinChunk ? n - c0 : kLinChunk);
-    const bool more = c0 + kLinChunk < n;
+  lay_s(s_lds);
+  lay_v(v_lds);
+  if (chunks > 1) fetch_v(1);
+  for (int c = 0; c < chunks; ++c) {
+    const bool more = c + 1 < chunks;
+    const uint8_t* v_in = v_lds + (c & 1) * V_BUF;
     fr += frag_step;
     keep += keep_step;
-    __syncthreads();                     // everyone is done with the tiles of the chunk in front
-    if (a.act) silu8(vr);
-    if (v_mine) *reinterpret_cast<uint4*>(v_lds + v_row * VS + v_e * 2) = vr.u;
-#pragma unroll
-    for (int dt = 0; dt < DTW; ++dt) {
-      const int d0 = 16 * (dt0 + dt) + 4 * g;
-#pragma unroll
-      for (int et = 0; et < ETW; ++et) {
-        uint2 hi, lo;
-        hi_lo(acc[dt][et][0], acc[dt][et][1], hi.x, lo.x);
-        hi_lo(acc[dt][et][2], acc[dt][et][3], hi.y, lo.y);
-        *reinterpret_cast<uint2*>(s_hi + (16 * (et0 + et) + r) * RS + d0 * 2) = hi;
-        *reinterpret_cast<uint2*>(s_lo + (16 * (et0 + et) + r) * RS + d0 * 2) = lo;
-      }
+    __syncthreads();                     // results of the chunk in front are done with the other two places
+    if (more) {
+      lay_v(v_lds + ((c + 1) & 1) * V_BUF);
+      if (c + 2 < chunks) fetch_v(c + 2);
     }
-    __syncthreads();
-    if (more) fetch_v(c0 + kLinChunk);
-    // o = S^T q, high and low parts; the operands of the next 32 elements are on their way out of LDS during a product
-    f32x4 o[ETO];
-#pragma unroll
-    for (int et = 0; et < ETO; ++et) o[et] = f32x4{0.f, 0.f, 0.f, 0.f};
-    {
-      Frag16 sa[2][ETO][2];
-      auto load = [&](int kk, Frag16 (&x)[ETO][2]) {
-#pragma unroll
-        for (int et = 0; et < ETO; ++et) {
-          const int off = (16 * (eto0 + et) + r) * RS + g * 16 + kk * 64;
-          x[et][0].u = *reinterpret_cast<const uint4*>(s_hi + off);
-          x[et][1].u = *reinterpret_cast<const uint4*>(s_lo + off);
-        }
-      };
-      load(0, sa[0]);
-#pragma unroll
-      for (int kk = 0; kk < ND; ++kk) {
-        if (kk + 1 < ND) load(kk + 1, sa[(kk + 1) & 1]);
-        __builtin_amdgcn_sched_barrier(0);
-        Frag16(&x)[ETO][2] = sa[kk & 1];
-#pragma unroll
-        for (int et = 0; et < ETO; ++et) o[et] = mma16<bf16_t>(x[et][0], qf[kk][0], o[et]);
-#pragma unroll
-        for (int et = 0; et < ETO; ++et) o[et] = mma16<bf16_t>(x[et][1], qf[kk][0], o[et]);
-#pragma unroll
-        for (int et = 0; et < ETO; ++et) o[et] = mma16<bf16_t>(x[et][0], qf[kk][1], o[et]);
-        __builtin_amdgcn_sched_barrier(0);
-      }
-    }
-    if (more) fetch_q(fr);
-    // the chunk's own tokens
-#pragma unroll
-    for (int s = 0; s < 2; ++s) {
-      if (2 * s > qt) break;
-#pragma unroll
-      for (int et = 0; et < ETO; ++et) {
-        const Frag16 v = transposed<VS>(v_lds, s, eto0 + et);
-        o[et] = mma16<bf16_t>(v, wf[s][0], o[et]);
-        o[et] = mma16<bf16_t>(v, wf[s][1], o[et]);
-      }
-    }
-    if (more) fetch_w(fr);
-    if (16 * qt + r < cnt) {
-      float* w = work + (c0 + 16 * qt + r) * a.wld;
-#pragma unroll
-      for (int et = 0; et < ETO; ++et) {
-        const int e = 16 * (eto0 + et) + 4 * g;
-        if (e0 + e < E) *reinterpret_cast<float4*>(w + e) =
-            float4{o[et][0] * a.q_scale, o[et][1] * a.q_scale, o[et][2] * a.q_scale, o[et][3] * a.q_scale};
-      }
-    }
-    // S <- diag(e^(b_last)) S + K^T V
 #pragma unroll
     for (int dt = 0; dt < DTW; ++dt)
 #pragma unroll
-      for (int et = 0; et < ETW; ++et) {
+      for (int et = 0; et < EC; ++et) {
         acc[dt][et][0] *= kp[dt].x;
         acc[dt][et][1] *= kp[dt].y;
         acc[dt][et][2] *= kp[dt].z;
@@ -679,19 +687,22 @@ __global__ void __launch_bounds__(512, 2) chunk_walk_kernel(LinArgs a) {
       }
 #pragma unroll
     for (int s = 0; s < 2; ++s) {
-      Frag16 v[ETW];
+      Frag16 v[EC];
 #pragma unroll
-      for (int et = 0; et < ETW; ++et) v[et] = transposed<VS>(v_lds, s, et0 + et);
-#pragma unroll
-      for (int dt = 0; dt < DTW; ++dt)
-#pragma unroll
-        for (int et = 0; et < ETW; ++et) acc[dt][et] = mma16<bf16_t>(kf[dt][s][0], v[et], acc[dt][et]);
+      for (int et = 0; et < EC; ++et) v[et] = transposed<VS, false>(v_in, s, et);
 #pragma unroll
       for (int dt = 0; dt < DTW; ++dt)
 #pragma unroll
-        for (int et = 0; et < ETW; ++et) acc[dt][et] = mma16<bf16_t>(kf[dt][s][1], v[et], acc[dt][et]);
+        for (int et = 0; et < EC; ++et) acc[dt][et] = mma16<bf16_t>(kf[dt][s][0], v[et], acc[dt][et]);
+#pragma unroll
+      for (int dt = 0; dt < DTW; ++dt)
+#pragma unroll
+        for (int et = 0; et < EC; ++et) acc[dt][et] = mma16<bf16_t>(kf[dt][s][1], v[et], acc[dt][et]);
     }
-    if (more) fetch_k(fr, keep);
+    if (more) {
+      fetch_k(fr, keep);
+      lay_s(s_lds + ((c + 1) & 1) * S_BUF);
+    }
   }
 #pragma unroll
   for (int dt = 0; dt < DTW; ++dt)
@@ -700,8 +711,8 @@ __global__ void __launch_bounds__(512, 2) chunk_walk_kernel(LinArgs a) {
       const int d = 16 * (dt0 + dt) + 4 * g + i;
       if (d >= D) continue;
 #pragma unroll
-      for (int et = 0; et < ETW; ++et) {
-        const int e = 16 * (et0 + et) + r;
+      for (int et = 0; et < EC; ++et) {
+        const int e = 16 * et + r;
         if (e0 + e < E) S[(int64_t)d * E + e] = acc[dt][et][i];
       }
     }
@@ -713,7 +724,17 @@ template <typename T>
 __device__ __forceinline__ float channel_decay(const LinArgs& a, const T* row, int64_t hd) {
   float z = a.a2_bias[hd];
   const T* w = (const T*)a.a2 + hd * a.rank;
-  for (int i = 0; i < a.rank; ++i) z += Elem<T>::to_f(row[a.a_off + i]) * Elem<T>::to_f(w[i]);
+  const T* x = row + a.a_off;
+  constexpr int V = Elem<T>::kVec;
+  if (a.rank % V == 0 && ((((uintptr_t)a.a2) | ((uintptr_t)x)) & 15) == 0) {
+    for (int i = 0; i < a.rank; i += V) {
+      const Vec16<T> wv = load16(w + i), xv = load16(x + i);
+#pragma unroll
+      for (int u = 0; u < V; ++u) z += Elem<T>::to_f(xv.e[u]) * Elem<T>::to_f(wv.e[u]);
+    }
+  } else {
+    for (int i = 0; i < a.rank; ++i) z += Elem<T>::to_f(x[i]) * Elem<T>::to_f(w[i]);
+  }
   return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * a.inv_tau);
 }
 template <typename T>
@@ -1017,9 +1038,9 @@ extern "C" int semipd_linear_attention(const void* proj, int64_t ld, int64_t q_o
       a.frags = reinterpret_cast<uint8_t*>(rest);
       a.keep = rest + chunks * num_heads * lin_frags(nd) * 256;
       const dim3 pgrid((unsigned)chunks, (unsigned)num_heads);
-      // 64 columns of S a workgroup where that leaves a workgroup for every CU, 32 otherwise
+      // one workgroup fits a CU: 32 columns of S each while they all run at once, 64 otherwise
       const int cus = owned_cus().load() > 0 ? owned_cus().load() : 256;
-      const bool wide = batch * num_heads * ((v_dim + 63) / 64) >= cus;
+      const bool wide = batch * num_heads * ((v_dim + 31) / 32) > cus;
       const int64_t items = batch * num_heads * ((v_dim + (wide ? 63 : 31)) / (wide ? 64 : 32));
       const dim3 wgrid((unsigned)((items + 7) / 8 * 8));
       static std::atomic<uint64_t> done[12] = {};
